@@ -815,7 +815,7 @@ int mi355_head_rmsnorm_gate_act(void* out, const float* o, const void* weight, c
  *   before t in its sequence), else 0 (before position 0).  w2 / y2: a second filter over the same input (null: none).
  *   act 0 none, 1 silu, 2 squared relu.  Without segments the launch also shifts the state; with segments
  *   mi355_causal_conv_state_update does, afterwards: the last taps - 1 of (old rows, the step's inputs).
- * mi355_activation: out[r][i] = act(in[r * in_stride + i]), act 1 or 2 as above. */
+ * mi355_activation: out[r][i] = act(in[r * in_stride + i]), act 1 or 2 as above, or 3 = erf-GELU. */
 int mi355_causal_conv(void* y1, void* y2, const void* u, int64_t u_stride, const void* w1, const void* w2, float* state,
                       const int32_t* req_to_state, const int64_t* req_pool_indices, const int32_t* tok_req,
                       const int32_t* seg_start, const int64_t* positions, int64_t tokens, int64_t channels, int taps,
@@ -926,6 +926,63 @@ int mi355_window_attention_pooled(void* out, const void* q, const void* k_cache,
                                   int64_t req_to_token_stride, int heads, int kv_heads, int head_dim, int v_head_dim, int window,
                                   int pool, int pool_div, float scale, int num_splits, float* split_scratch, int64_t tokens,
                                   int max_run, int dtype, void* stream);
+
+/* ---- latent attention over every earlier token, in either rotation pairing ----------------------------------
+ * mi355_latent_rows_write: mi355_latent_norms_rope_write where the leading q_cols columns may be left alone (cq and q_weight
+ *   null: queries that are not normed), the rotation pairs feature i with i + rot_dims / 2 or (interleaved) 2 i with 2 i + 1,
+ *   and cos and sin are multiplied by rot_mag.
+ * mi355_latent_attention: mi355_latent_window_attention with the same rotation of qr, window 0 = every earlier token, and
+ *   sink null = a plain softmax. */
+int mi355_latent_rows_write(void* cq, void* cache, const void* a, const void* q_weight, const void* kv_weight,
+                            const int64_t* positions, const int64_t* out_cache_loc, const float* inv_freq, int64_t tokens,
+                            int64_t a_stride, int q_cols, int rank, int rope_dim, int rot_dims, int interleaved, float rot_mag,
+                            int64_t num_slots, float eps, int dtype, void* stream);
+int mi355_latent_attention(void* out, const void* qa, const void* qr, const void* cache, const void* gate,
+                           const int32_t* req_to_token, const int64_t* req_pool_indices, const int32_t* tok_req,
+                           const int64_t* positions, const int32_t* blocks, int64_t num_blocks, const float* sink,
+                           const float* inv_freq, int64_t qa_token_stride, int64_t qa_head_stride, int64_t qr_token_stride,
+                           int64_t qr_head_stride, int64_t out_token_stride, int64_t out_head_stride, int64_t gate_stride,
+                           int64_t req_to_token_stride, int heads, int rank, int rope_dim, int rot_dims, int interleaved,
+                           float rot_mag, int window, float scale, int num_splits, float* split_scratch, int64_t tokens, int dtype,
+                           void* stream);
+
+/* ---- matrix memory with exponential gates ----------------------------------------------------------------
+ * Per head over every sequence's tokens of the step, all gates, q_scale, state and results fp32:
+ *   i = c tanh((in_logits[t, h] + in_bias[h]) / c),  f = logsigmoid(c tanh((forget_logits[t, h] + forget_bias[h]) / c)),  c = gate_cap
+ *   m' = max(f + m, i);  S <- e^(f + m - m') S + e^(i - m') k v^T;  n <- e^(f + m - m') n + e^(i - m') k;  m <- m'
+ *   out[t, h] = S^T q / (max(|n . q|, e^-m) + 1e-6),  q = q_scale * q[t, h]
+ * state [slots, heads, key_dim, value_dim]; norm_state [slots, heads, norm_blocks, key_dim + 1] holds (n, m) once per
+ * mi355_matrix_memory_value_block() value columns (norm_blocks = their number, rounded up).  A sequence at position 0 starts
+ * from zeros, any other from its slot.  Segments as mi355_linear_recurrence.  key_dim <= 256. */
+int mi355_matrix_memory_value_block(void);
+int mi355_matrix_memory(float* out, float* state, float* norm_state, const void* q, const void* k, const void* v,
+                        const float* in_logits, const float* forget_logits, const float* in_bias, const float* forget_bias,
+                        const int32_t* req_to_state, const int64_t* req_pool_indices, const int32_t* seg_start, const int32_t* seg_len,
+                        const int64_t* positions, int64_t batch, int heads, int key_dim, int value_dim, int norm_blocks,
+                        int64_t q_token_stride, int64_t k_token_stride, int64_t v_token_stride, int64_t gate_token_stride,
+                        float q_scale, float gate_cap, int dtype, void* stream);
+/* mi355_head_rmsnorm_gate_wide: mi355_head_rmsnorm_gate_act with a weight of its own per head ([heads][value_dim]) if
+ *   weight_per_head. */
+int mi355_head_rmsnorm_gate_wide(void* out, const float* o, const void* weight, int weight_per_head, const void* gate, int64_t gate_stride,
+                                 int64_t tokens, int heads, int value_dim, float eps, int gate_act, int dtype, void* stream);
+
+/* ---- layer norms around every sublayer of an fp32 stream, clamped gated experts ------------------------------------
+ * mi355_layernorm_residual_add: x[t] += LN(b) * w_out in place, then h[t] = LN(x[t]) * w_next in the activation dtype (w_next
+ *   and h null: not), LN the layer norm (y - mean) / sqrt(mean of squared deviations + eps), b = sum_j y[rows[t * n_rows + j]]
+ *   (rows null: y[t]) + sigmoid(y2_gate[t * gate_stride]) * y2[t] (y2 null: nothing).
+ * mi355_project_f32: out[t][n] = x[t] . weight[n] in unrounded fp32 (16-bit operands, out contiguous).
+ * mi355_moe_route_scores_strided: mi355_moe_route_scores on rows of logits that lie logit_stride apart.
+ * mi355_clamped_glu: out[p][i] = g sigmoid(alpha g) (u + 1), g = min(c a[p][i], limit), u = clamp(c a[p][ff + i], -limit, limit),
+ *   for the `pairs` rows p = rows[j] (rows null: p = j), c = coef[j] (coef null: 1); other rows of out are left alone. */
+int mi355_layernorm_residual_add(float* x, void* h, const void* y, int64_t y_stride, const int32_t* rows, int n_rows, const void* y2,
+                                 int64_t y2_stride, const float* y2_gate, int64_t gate_stride, const void* w_out, const void* w_next,
+                                 int64_t tokens, int64_t hidden, float eps, int dtype, void* stream);
+int mi355_project_f32(float* out, const void* x, int64_t x_stride, const void* weight, int64_t rows, int n, int k, int dtype, void* stream);
+int mi355_moe_route_scores_strided(int32_t* ids, float* weights, const float* logits, int64_t logit_stride, const float* correction,
+                                   int64_t tokens, int num_experts, int top, int n_groups, int keep_groups, float scale, int score_fn,
+                                   int group_best, int renorm, void* stream);
+int mi355_clamped_glu(void* out, const void* a, int64_t a_stride, const int32_t* rows, const float* coef, int64_t pairs, int ff,
+                      float limit, float alpha, int dtype, void* stream);
 
 #ifdef __cplusplus
 }

@@ -137,6 +137,15 @@ _SIGNATURES = {
     "mi355_pool_kv_blocks": (I, [P, P, P, P, P, P, P, P, L, L, I, I, I, I, I, I, P]),
     "mi355_window_attention_pooled": (I, [P, P, P, P, P, P, P, P, P, P, P, L, P, P, L, L, L, L, L, L, I, I, I, I, I, I, I, F, I, P, L, I, I, P]),
     "mi355_latent_window_attention": (I, [P, P, P, P, P, P, P, P, P, P, L, P, P, L, L, L, L, L, L, L, L, I, I, I, I, I, F, I, P, L, I, P]),
+    "mi355_latent_rows_write": (I, [P, P, P, P, P, P, P, P, L, L, I, I, I, I, I, F, L, F, I, P]),
+    "mi355_latent_attention": (I, [P, P, P, P, P, P, P, P, P, P, L, P, P, L, L, L, L, L, L, L, L, I, I, I, I, I, F, I, F, I, P, L, I, P]),
+    "mi355_matrix_memory_value_block": (I, []),
+    "mi355_matrix_memory": (I, [P, P, P, P, P, P, P, P, P, P, P, P, P, P, P, L, I, I, I, I, L, L, L, L, F, F, I, P]),
+    "mi355_head_rmsnorm_gate_wide": (I, [P, P, P, I, P, L, L, I, I, F, I, I, P]),
+    "mi355_layernorm_residual_add": (I, [P, P, P, L, P, I, P, L, P, L, P, P, L, L, F, I, P]),
+    "mi355_project_f32": (I, [P, P, L, P, L, I, I, I, P]),
+    "mi355_moe_route_scores_strided": (I, [P, P, P, L, P, L, I, I, I, I, F, I, I, I, P]),
+    "mi355_clamped_glu": (I, [P, P, L, P, P, L, I, F, F, I, P]),
 }
 
 EXPORTED_SYMBOLS = tuple(_SIGNATURES)

@@ -1,10 +1,13 @@
-// Sliding-window attention over a latent KV cache, with a learned sink in the softmax denominator.
+// Attention over a latent KV cache: the last `window` tokens or (window 0) every earlier one, with or without a learned sink
+// in the softmax denominator.
 //
 // The cache holds one row per token and layer: [ c (rank features) | k_r (rope features, already rotated) ].  In the
 // absorbed form every head h attends the same rows: score(t, j) = (qa[t,h] . c[j] + rot(qr[t,h]) . k_r[j]) * scale
-// with qa = q_nope W_uk[h], and the result per head is sum_j p(t, j) c[j] (the caller applies W_uv[h]).  Query at
+// with qa = q_nope W_uk[h], and the result per head is sum_j p(t, j) c[j] (the caller applies W_uv[h]).  rot turns feature
+// pairs (i, i + n / 2), or (2 i, 2 i + 1) when interleaved, with cos and sin times a magnitude.  Query at
 // position p sees key j iff 0 <= p - j < window.  softmax: p(t, j) = exp(s_j - m) / (sum_j exp(s_j - m) + exp(sink_h - m));
-// the sink has no value row, so the running (max, sum) pair simply starts at (sink_h, 1).
+// the sink has no value row, so the running (max, sum) pair simply starts at (sink_h, 1) -- or, without a sink, at (a very
+// low finite number, 0).
 //
 //   mi355_latent_norms_rope_write   the step before it: both latent RMS norms of the "a" projection's row, the
 //                                   rotation of the shared rope key and the write of the cache row
@@ -18,24 +21,33 @@
 namespace mi355 {
 namespace {
 
+constexpr float LATENT_NO_SINK = -1e30f;      // start of a running maximum without a sink: finite, so that a tile without visible keys is harmless
+
+// features of rotation pair i among the first rot_dims of a vector
+__device__ __forceinline__ int rot_first(int i, int interleaved) { return interleaved ? 2 * i : i; }
+__device__ __forceinline__ int rot_second(int i, int half, int interleaved) { return interleaved ? 2 * i + 1 : i + half; }
+
 // ------------------------------------------------------------------------------------------ latent norms + rope + cache write
-// One workgroup per token.  a[t] = [ q latent (q_rank) | kv latent (rank) | rope key (dr) | ... ].
+// One workgroup per token.  a[t] = [ q latent (q_rank) | kv latent (rank) | rope key (dr) | ... ].  cq null: the first q_rank
+// columns are whatever the caller keeps there (queries that are not normed) and are left alone.
 template <typename T>
 __global__ __launch_bounds__(256) void latent_norms_rope_write_kernel(
     T* __restrict__ cq, T* __restrict__ cache, const T* __restrict__ a, const T* __restrict__ wq, const T* __restrict__ wkv,
     const int64_t* __restrict__ positions, const int64_t* __restrict__ loc, const float* __restrict__ inv_freq, int64_t a_stride,
-    int q_rank, int rank, int dr, int rot_dims, float eps) {
+    int q_rank, int rank, int dr, int rot_dims, int interleaved, float rot_mag, float eps) {
   __shared__ float red[16];
   const int64_t t = blockIdx.x;
   const T* row = a + t * a_stride;
   float s = 0.f;
-  for (int i = threadIdx.x; i < q_rank; i += blockDim.x) {
-    const float v = to_f32(row[i]);
-    s += v * v;
+  if (cq != nullptr) {
+    for (int i = threadIdx.x; i < q_rank; i += blockDim.x) {
+      const float v = to_f32(row[i]);
+      s += v * v;
+    }
+    const float inv_q = 1.0f / sqrtf(block_sum(s, red) / (float)q_rank + eps);
+    for (int i = threadIdx.x; i < q_rank; i += blockDim.x) cq[t * q_rank + i] = from_f32<T>(to_f32(row[i]) * inv_q * to_f32(wq[i]));
+    s = 0.f;
   }
-  const float inv_q = 1.0f / sqrtf(block_sum(s, red) / (float)q_rank + eps);
-  for (int i = threadIdx.x; i < q_rank; i += blockDim.x) cq[t * q_rank + i] = from_f32<T>(to_f32(row[i]) * inv_q * to_f32(wq[i]));
-  s = 0.f;
   for (int i = threadIdx.x; i < rank; i += blockDim.x) {
     const float v = to_f32(row[q_rank + i]);
     s += v * v;
@@ -49,9 +61,12 @@ __global__ __launch_bounds__(256) void latent_norms_rope_write_kernel(
   for (int i = threadIdx.x; i < half; i += blockDim.x) {
     float sn, cs;
     sincosf(pos * inv_freq[i], &sn, &cs);
-    const float u = to_f32(kr[i]), v = to_f32(kr[i + half]);
-    dst[rank + i] = from_f32<T>(u * cs - v * sn);
-    dst[rank + i + half] = from_f32<T>(v * cs + u * sn);
+    sn *= rot_mag;
+    cs *= rot_mag;
+    const int ia = rot_first(i, interleaved), ib = rot_second(i, half, interleaved);
+    const float u = to_f32(kr[ia]), v = to_f32(kr[ib]);
+    dst[rank + ia] = from_f32<T>(u * cs - v * sn);
+    dst[rank + ib] = from_f32<T>(v * cs + u * sn);
   }
   for (int i = rot_dims + threadIdx.x; i < dr; i += blockDim.x) dst[rank + i] = kr[i];
 }
@@ -68,11 +83,11 @@ struct LatentAttnParams {
   const int32_t* tok_req;     // null: token t belongs to sequence t
   const int64_t* positions;
   const int32_t* blocks;      // pairs (first token, count) of runs inside one sequence, or null: one token per run
-  const float* sink;          // [H]
+  const float* sink;          // [H], or null
   const float* inv_freq;      // [rot_dims / 2]
   int64_t qa_st, qa_sh, qr_st, qr_sh, o_st, o_sh, gate_st, rtt_stride;
-  int H, rank, dr, rot_dims, window, hg, kb, rows_cap;
-  float scale;
+  int H, rank, dr, rot_dims, window, hg, kb, rows_cap, interleaved;
+  float scale, rot_mag;
   // matrix-core kernel only: the keys of a run cut into nsplit ranges, one workgroup each; unnormalised partial
   // sums, maxima and denominators go to part_o / part_m / part_l ([nsplit][tokens][H][...]) for the merge kernel
   int nsplit;
@@ -154,9 +169,12 @@ __global__ __launch_bounds__(256) void latent_window_attention_kernel(const Late
     const T* src = qr + (int64_t)(t0 + ti) * p.qr_st + (int64_t)(h0 + hi) * p.qr_sh;
     float sn, cs;
     sincosf((float)(p0 + ti) * p.inv_freq[i], &sn, &cs);
-    const float u = to_f32(src[i]), v = to_f32(src[i + half]);
-    Q[(size_t)m * rp + rank + i] = u * cs - v * sn;
-    Q[(size_t)m * rp + rank + i + half] = v * cs + u * sn;
+    sn *= p.rot_mag;
+    cs *= p.rot_mag;
+    const int ia = rot_first(i, p.interleaved), ib = rot_second(i, half, p.interleaved);
+    const float u = to_f32(src[ia]), v = to_f32(src[ib]);
+    Q[(size_t)m * rp + rank + ia] = u * cs - v * sn;
+    Q[(size_t)m * rp + rank + ib] = v * cs + u * sn;
   }
   const int tail = dr - p.rot_dims;
   for (int idx = tid; idx < M * tail; idx += nt) {
@@ -166,8 +184,8 @@ __global__ __launch_bounds__(256) void latent_window_attention_kernel(const Late
   }
   for (int idx = tid; idx < M * rank; idx += nt) O[idx] = 0.f;
   for (int m = tid; m < M; m += nt) {
-    mrow[m] = p.sink[h0 + (m % nh)];
-    lrow[m] = 1.0f;
+    mrow[m] = p.sink ? p.sink[h0 + (m % nh)] : LATENT_NO_SINK;
+    lrow[m] = p.sink ? 1.0f : 0.0f;
   }
   __syncthreads();
 
@@ -344,9 +362,12 @@ __global__ __launch_bounds__(256) void latent_window_attention_mfma_kernel(const
       for (int i = lane; i < half; i += 64) {
         float sn, cs;
         sincosf(pos * p.inv_freq[i], &sn, &cs);
-        const float u = to_f32(rs[i]), w = to_f32(rs[i + half]);
-        dst[rank + i] = from_f32<T>(u * cs - w * sn);
-        dst[rank + i + half] = from_f32<T>(w * cs + u * sn);
+        sn *= p.rot_mag;
+        cs *= p.rot_mag;
+        const int ia = rot_first(i, p.interleaved), ib = rot_second(i, half, p.interleaved);
+        const float u = to_f32(rs[ia]), w = to_f32(rs[ib]);
+        dst[rank + ia] = from_f32<T>(u * cs - w * sn);
+        dst[rank + ib] = from_f32<T>(w * cs + u * sn);
       }
       for (int i = p.rot_dims + lane; i < dr; i += 64) dst[rank + i] = rs[i];
       for (int r = R + lane; r < RP; r += 64) dst[r] = from_f32<T>(0.f);
@@ -364,8 +385,8 @@ __global__ __launch_bounds__(256) void latent_window_attention_mfma_kernel(const
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
     const int m = r0 + 4 * lg + r;
-    const bool with_sink = split == 0 && m < M;
-    mrun[r] = with_sink ? p.sink[h0 + (m % nh)] * 1.4426950408889634f : -1e30f;     // base-2 units, as the scores
+    const bool with_sink = split == 0 && m < M && p.sink != nullptr;
+    mrun[r] = with_sink ? p.sink[h0 + (m % nh)] * 1.4426950408889634f : LATENT_NO_SINK;     // base-2 units, as the scores
     lrun[r] = with_sink ? 1.0f : 0.0f;
   }
   f32x4 acc[RT][CT];
@@ -646,18 +667,29 @@ int mi355_latent_norms_rope_write(void* cq, void* cache, const void* a, const vo
                                   const int64_t* positions, const int64_t* out_cache_loc, const float* inv_freq, int64_t tokens,
                                   int64_t a_stride, int q_rank, int rank, int rope_dim, int rot_dims, int64_t num_slots, float eps,
                                   int dtype, void* stream) {
-  MI355_REQUIRE(cq && cache && a && q_weight && kv_weight && positions && out_cache_loc && inv_freq, MI355_ERR_INVALID,
-                "latent_norms_rope_write: null pointer");
-  MI355_REQUIRE(tokens >= 0 && q_rank > 0 && rank > 0 && rope_dim >= 0 && rot_dims >= 0 && rot_dims <= rope_dim && rot_dims % 2 == 0 &&
-                    a_stride >= (int64_t)q_rank + rank + rope_dim && num_slots > 0,
-                MI355_ERR_INVALID, "latent_norms_rope_write: bad shape");
+  MI355_REQUIRE(cq && q_weight && q_rank > 0, MI355_ERR_INVALID, "latent_norms_rope_write: null pointer");
+  return mi355_latent_rows_write(cq, cache, a, q_weight, kv_weight, positions, out_cache_loc, inv_freq, tokens, a_stride, q_rank, rank,
+                                 rope_dim, rot_dims, 0, 1.0f, num_slots, eps, dtype, stream);
+}
+
+int mi355_latent_rows_write(void* cq, void* cache, const void* a, const void* q_weight, const void* kv_weight,
+                            const int64_t* positions, const int64_t* out_cache_loc, const float* inv_freq, int64_t tokens,
+                            int64_t a_stride, int q_cols, int rank, int rope_dim, int rot_dims, int interleaved, float rot_mag,
+                            int64_t num_slots, float eps, int dtype, void* stream) {
+  MI355_REQUIRE(cache && a && kv_weight && positions && out_cache_loc && (rot_dims == 0 || inv_freq), MI355_ERR_INVALID,
+                "latent_rows_write: null pointer");
+  MI355_REQUIRE((cq == nullptr) == (q_weight == nullptr) && (cq == nullptr || q_cols > 0), MI355_ERR_INVALID,
+                "latent_rows_write: the normed queries, their weight and their columns come together");
+  MI355_REQUIRE(tokens >= 0 && q_cols >= 0 && rank > 0 && rope_dim >= 0 && rot_dims >= 0 && rot_dims <= rope_dim && rot_dims % 2 == 0 &&
+                    a_stride >= (int64_t)q_cols + rank + rope_dim && num_slots > 0,
+                MI355_ERR_INVALID, "latent_rows_write: bad shape");
   if (tokens == 0) return MI355_OK;
-  MI355_DISPATCH_DTYPE(dtype, "latent_norms_rope_write", {
+  MI355_DISPATCH_DTYPE(dtype, "latent_rows_write", {
     hipLaunchKernelGGL((latent_norms_rope_write_kernel<T>), dim3((unsigned)tokens), dim3(256), 0, (hipStream_t)stream, (T*)cq,
                        (T*)cache, (const T*)a, (const T*)q_weight, (const T*)kv_weight, positions, out_cache_loc, inv_freq, a_stride,
-                       q_rank, rank, rope_dim, rot_dims, eps);
+                       q_cols, rank, rope_dim, rot_dims, interleaved, rot_mag, eps);
   });
-  MI355_CHECK_LAUNCH("latent_norms_rope_write");
+  MI355_CHECK_LAUNCH("latent_rows_write");
   return MI355_OK;
 }
 
@@ -675,16 +707,31 @@ int mi355_latent_window_attention(void* out, const void* qa, const void* qr, con
                                   int64_t qr_head_stride, int64_t out_token_stride, int64_t out_head_stride, int64_t gate_stride,
                                   int64_t req_to_token_stride, int heads, int rank, int rope_dim, int rot_dims, int window,
                                   float scale, int num_splits, float* split_scratch, int64_t tokens, int dtype, void* stream) {
-  MI355_REQUIRE(out && qa && cache && req_to_token && req_pool_indices && positions && sink, MI355_ERR_INVALID,
-                "latent_window_attention: null pointer");
-  MI355_REQUIRE(rope_dim == 0 || (qr && inv_freq), MI355_ERR_INVALID, "latent_window_attention: the rope part needs qr and inv_freq");
-  MI355_REQUIRE(heads > 0 && rank > 0 && rope_dim >= 0 && rot_dims >= 0 && rot_dims <= rope_dim && rot_dims % 2 == 0 && window > 0 &&
+  MI355_REQUIRE(sink && window > 0, MI355_ERR_INVALID, "latent_window_attention: needs a sink and a window");
+  return mi355_latent_attention(out, qa, qr, cache, gate, req_to_token, req_pool_indices, tok_req, positions, blocks, num_blocks, sink,
+                                inv_freq, qa_token_stride, qa_head_stride, qr_token_stride, qr_head_stride, out_token_stride,
+                                out_head_stride, gate_stride, req_to_token_stride, heads, rank, rope_dim, rot_dims, 0, 1.0f, window,
+                                scale, num_splits, split_scratch, tokens, dtype, stream);
+}
+
+int mi355_latent_attention(void* out, const void* qa, const void* qr, const void* cache, const void* gate,
+                           const int32_t* req_to_token, const int64_t* req_pool_indices, const int32_t* tok_req,
+                           const int64_t* positions, const int32_t* blocks, int64_t num_blocks, const float* sink,
+                           const float* inv_freq, int64_t qa_token_stride, int64_t qa_head_stride, int64_t qr_token_stride,
+                           int64_t qr_head_stride, int64_t out_token_stride, int64_t out_head_stride, int64_t gate_stride,
+                           int64_t req_to_token_stride, int heads, int rank, int rope_dim, int rot_dims, int interleaved,
+                           float rot_mag, int window, float scale, int num_splits, float* split_scratch, int64_t tokens, int dtype,
+                           void* stream) {
+  MI355_REQUIRE(out && qa && cache && req_to_token && req_pool_indices && positions, MI355_ERR_INVALID,
+                "latent_attention: null pointer");
+  MI355_REQUIRE((rope_dim == 0 || qr) && (rot_dims == 0 || inv_freq), MI355_ERR_INVALID, "latent_attention: the rope part needs qr and inv_freq");
+  MI355_REQUIRE(heads > 0 && rank > 0 && rope_dim >= 0 && rot_dims >= 0 && rot_dims <= rope_dim && rot_dims % 2 == 0 && window >= 0 &&
                     num_blocks >= 0 && num_blocks < (1ll << 31),
-                MI355_ERR_INVALID, "latent_window_attention: bad shape");
+                MI355_ERR_INVALID, "latent_attention: bad shape");
   if (num_blocks == 0) return MI355_OK;
   const bool mfma = latent_mfma_serves(dtype, rank, rope_dim);
   MI355_REQUIRE(num_splits >= 1 && num_splits <= 64 && (num_splits == 1 || (mfma && blocks == nullptr && split_scratch && tokens == num_blocks)),
-                MI355_ERR_INVALID, "latent_window_attention: key splits need the 16-bit kernel, one token per run and a scratch array");
+                MI355_ERR_INVALID, "latent_attention: key splits need the 16-bit kernel, one token per run and a scratch array");
   LatentAttnPlan pl = plan_latent_attn(heads, rank, rope_dim);
   if (mfma) {
     pl.hg = std::min(heads, LM_ROWS);
@@ -692,7 +739,7 @@ int mi355_latent_window_attention(void* out, const void* qa, const void* qr, con
     pl.kb = LM_KB;
     pl.lds = lm_lds_bytes(rank, rope_dim);
   }
-  MI355_REQUIRE(pl.lds <= 160 * 1024, MI355_ERR_UNSUPPORTED, "latent_window_attention: rank %d + rope %d does not fit the LDS tile", rank,
+  MI355_REQUIRE(pl.lds <= 160 * 1024, MI355_ERR_UNSUPPORTED, "latent_attention: rank %d + rope %d does not fit the LDS tile", rank,
                 rope_dim);
   LatentAttnParams p;
   p.qa = qa; p.qr = qr; p.out = out; p.cache = cache; p.gate = gate;
@@ -700,8 +747,9 @@ int mi355_latent_window_attention(void* out, const void* qa, const void* qr, con
   p.blocks = blocks; p.sink = sink; p.inv_freq = inv_freq;
   p.qa_st = qa_token_stride; p.qa_sh = qa_head_stride; p.qr_st = qr_token_stride; p.qr_sh = qr_head_stride;
   p.o_st = out_token_stride; p.o_sh = out_head_stride; p.gate_st = gate_stride; p.rtt_stride = req_to_token_stride;
-  p.H = heads; p.rank = rank; p.dr = rope_dim; p.rot_dims = rot_dims; p.window = window; p.hg = pl.hg; p.kb = pl.kb; p.rows_cap = pl.hg * pl.bq;
-  p.scale = scale;
+  p.H = heads; p.rank = rank; p.dr = rope_dim; p.rot_dims = rot_dims; p.hg = pl.hg; p.kb = pl.kb; p.rows_cap = pl.hg * pl.bq;
+  p.window = window > 0 ? window : 0x7fffffff;      // 0: every earlier token
+  p.scale = scale; p.interleaved = interleaved; p.rot_mag = rot_mag;
   p.nsplit = num_splits; p.tokens = tokens;
   p.part_o = split_scratch;
   p.part_m = split_scratch ? split_scratch + (int64_t)num_splits * tokens * heads * rank : nullptr;
@@ -712,22 +760,22 @@ int mi355_latent_window_attention(void* out, const void* qa, const void* qr, con
     const int rows = blocks == nullptr ? pl.hg : pl.hg * pl.bq;     // one token per run: a workgroup holds at most hg rows
     if (dtype == MI355_BF16) ok = launch_latent_mfma<bf16_t>(p, mgrid, rows, (hipStream_t)stream);
     else ok = launch_latent_mfma<f16_t>(p, mgrid, rows, (hipStream_t)stream);
-    MI355_REQUIRE(ok, MI355_ERR_UNSUPPORTED, "latent_window_attention: rank %d is not served", rank);
-    MI355_CHECK_LAUNCH("latent_window_attention");
+    MI355_REQUIRE(ok, MI355_ERR_UNSUPPORTED, "latent_attention: rank %d is not served", rank);
+    MI355_CHECK_LAUNCH("latent_attention");
     if (num_splits > 1) {
       const dim3 g2((unsigned)tokens, (unsigned)heads);
       if (dtype == MI355_BF16) hipLaunchKernelGGL((latent_window_merge_kernel<bf16_t>), g2, dim3(128), 0, (hipStream_t)stream, p);
       else hipLaunchKernelGGL((latent_window_merge_kernel<f16_t>), g2, dim3(128), 0, (hipStream_t)stream, p);
-      MI355_CHECK_LAUNCH("latent_window_attention (merge)");
+      MI355_CHECK_LAUNCH("latent_attention (merge)");
     }
     return MI355_OK;
   }
   const dim3 grid((unsigned)num_blocks, (unsigned)((heads + pl.hg - 1) / pl.hg), 1);
-  MI355_DISPATCH_DTYPE(dtype, "latent_window_attention", {
+  MI355_DISPATCH_DTYPE(dtype, "latent_attention", {
     auto kern = latent_window_attention_kernel<T>;
     if (pl.lds > 48 * 1024) (void)hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)pl.lds);
     hipLaunchKernelGGL(kern, grid, dim3(256), pl.lds, (hipStream_t)stream, p);
   });
-  MI355_CHECK_LAUNCH("latent_window_attention");
+  MI355_CHECK_LAUNCH("latent_attention");
   return MI355_OK;
 }

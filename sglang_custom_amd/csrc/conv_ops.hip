@@ -21,6 +21,7 @@ constexpr int CONV_MAX_TAPS = 8;
 __device__ __forceinline__ float conv_act(float z, int act) {
   if (act == 1) return z / (1.0f + expf(-z));
   if (act == 2) { const float r = fmaxf(z, 0.f); return r * r; }
+  if (act == 3) return 0.5f * z * (1.0f + erff(z * 0.7071067811865476f));
   return z;
 }
 
@@ -214,13 +215,19 @@ __global__ __launch_bounds__(256) void causal_conv_state_update_kernel(float* __
   }
 }
 
-template <typename T>
+// grid (column blocks, rows); VEC: eight 16-bit features per access
+template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void activation_kernel(T* __restrict__ out, const T* __restrict__ in, int64_t in_stride,
                                                          int64_t rows, int64_t cols, int act) {
-  const int64_t n = rows * cols;
-  for (int64_t idx = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; idx < n; idx += (int64_t)gridDim.x * blockDim.x) {
-    const int64_t r = idx / cols, i = idx - r * cols;
-    out[idx] = from_f32<T>(conv_act(to_f32(in[r * in_stride + i]), act));
+  constexpr int W = VEC ? 8 : 1;
+  for (int64_t r = blockIdx.y; r < rows; r += gridDim.y) {
+    for (int64_t i = W * ((int64_t)blockIdx.x * 256 + threadIdx.x); i < cols; i += W * 256 * (int64_t)gridDim.x) {
+      const Vec<T, W> v = ldvec<T, W>(in + r * in_stride + i);
+      Vec<T, W> o;
+#pragma unroll
+      for (int k = 0; k < W; ++k) o.v[k] = from_f32<T>(conv_act(to_f32(v.v[k]), act));
+      stvec<T, W>(out + r * cols + i, o);
+    }
   }
 }
 
@@ -299,12 +306,17 @@ int mi355_causal_conv_state_update(float* state, const void* u, int64_t u_stride
 
 int mi355_activation(void* out, const void* in, int64_t in_stride, int64_t rows, int64_t cols, int act, int dtype, void* stream) {
   MI355_REQUIRE(out && in, MI355_ERR_INVALID, "activation: null pointer");
-  MI355_REQUIRE(rows >= 0 && cols > 0 && in_stride >= cols && (act == 1 || act == 2), MI355_ERR_INVALID, "activation: bad shape or kind");
+  MI355_REQUIRE(rows >= 0 && cols > 0 && in_stride >= cols && act >= 1 && act <= 3, MI355_ERR_INVALID, "activation: bad shape or kind");
   if (rows == 0) return MI355_OK;
-  const int grid = (int)std::min<int64_t>((rows * cols + 255) / 256, 256 * 16);
+  const bool vec = dtype != MI355_F32 && cols % 8 == 0 && in_stride % 8 == 0 && aligned16(out) && aligned16(in);
+  const dim3 grid((unsigned)std::min<int64_t>((cols + (vec ? 2047 : 255)) / (vec ? 2048 : 256), 1024), (unsigned)std::min<int64_t>(rows, 65535));
   MI355_DISPATCH_DTYPE(dtype, "activation", {
-    hipLaunchKernelGGL((activation_kernel<T>), dim3(grid), dim3(256), 0, (hipStream_t)stream, (T*)out, (const T*)in, in_stride, rows,
-                       cols, act);
+    if (vec)
+      hipLaunchKernelGGL((activation_kernel<T, true>), grid, dim3(256), 0, (hipStream_t)stream, (T*)out, (const T*)in, in_stride, rows,
+                         cols, act);
+    else
+      hipLaunchKernelGGL((activation_kernel<T, false>), grid, dim3(256), 0, (hipStream_t)stream, (T*)out, (const T*)in, in_stride, rows,
+                         cols, act);
   });
   MI355_CHECK_LAUNCH("activation");
   return MI355_OK;

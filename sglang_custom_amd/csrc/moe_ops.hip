@@ -7,7 +7,9 @@
 //     through the sorted list (first GEMM) or taken in place (second GEMM); blocks past the used count exit at once.
 //     16-bit dtypes with K a multiple of 8 run on the matrix cores, reading both operands' fragments straight from
 //     global memory (a weight row and an input row are both contiguous along K, which is the fragment's direction);
-//     everything else (fp32: exact) on the vector ALU through LDS tiles.
+//     everything else (fp32: exact) on the vector ALU through LDS tiles,
+//   * mi355_project_f32: unrounded fp32 products of 16-bit rows with a small 16-bit table (router and gate logits),
+//   * mi355_clamped_glu: the clamped gated unit between an expert's two GEMMs, with the token's weight on the expert's INPUT.
 #include "common.cuh"
 
 #include <algorithm>
@@ -23,8 +25,8 @@ __device__ __forceinline__ float moe_gelu_erf(float z) { return 0.5f * z * (1.0f
 // One wave per token; sm per wave: choice[E] | score[E] | group[G]
 __global__ __launch_bounds__(256) void moe_route_grouped_kernel(int32_t* __restrict__ ids, float* __restrict__ weights,
                                                                 const float* __restrict__ logits,
-                                                                const float* __restrict__ correction, int64_t tokens, int E,
-                                                                int top, int n_groups, int keep, float scale, int score_fn,
+                                                                int64_t logit_stride, const float* __restrict__ correction,
+                                                                int64_t tokens, int E, int top, int n_groups, int keep, float scale, int score_fn,
                                                                 int group_best, int renorm) {
   extern __shared__ float sm[];
   const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
@@ -39,14 +41,14 @@ __global__ __launch_bounds__(256) void moe_route_grouped_kernel(int32_t* __restr
     if (score_fn == 1) {
       // softmax over all experts
       mx = -INFINITY;
-      for (int e = lane; e < E; e += 64) mx = fmaxf(mx, logits[t * E + e]);
+      for (int e = lane; e < E; e += 64) mx = fmaxf(mx, logits[t * logit_stride + e]);
       mx = wave_max(mx);
       float sum = 0.f;
-      for (int e = lane; e < E; e += 64) sum += expf(logits[t * E + e] - mx);
+      for (int e = lane; e < E; e += 64) sum += expf(logits[t * logit_stride + e] - mx);
       inv = 1.0f / wave_sum(sum);
     }
     for (int e = lane; e < E; e += 64) {
-      const float s = score_fn == 1 ? expf(logits[t * E + e] - mx) * inv : 1.0f / (1.0f + expf(-logits[t * E + e]));
+      const float s = score_fn == 1 ? expf(logits[t * logit_stride + e] - mx) * inv : 1.0f / (1.0f + expf(-logits[t * logit_stride + e]));
       score[e] = s;
       choice[e] = s + (correction != nullptr ? correction[e] : 0.f);
     }
@@ -440,6 +442,82 @@ __global__ __launch_bounds__(256) void moe_router_logits_kernel(float* __restric
   }
 }
 
+// Unrounded fp32 products of few table rows: out[t][n] = x[t] . w[n] with T operands (a product of two 16-bit numbers is exact
+// in fp32).  A workgroup takes a 16 x 16 tile of the result; its eight waves walk every eighth 32-wide step of K on the matrix
+// cores and meet in LDS, in a fixed order whatever the number of rows.
+constexpr int PJ_WAVES = 8;
+template <typename T>
+__global__ __launch_bounds__(64 * PJ_WAVES) void project_f32_mfma_kernel(float* __restrict__ out, const T* __restrict__ x, int64_t x_stride,
+                                                                        const T* __restrict__ w, int64_t rows, int N, int K) {
+  using Frag = typename Mfma<T>::frag;
+  __shared__ __attribute__((aligned(16))) f32x4 part[PJ_WAVES][64];
+  const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, li = lane & 15, lg = lane >> 4;
+  const int64_t t = (int64_t)blockIdx.x * 16 + li;
+  const int n = blockIdx.y * 16 + li;
+  // rows past either end read row 0; their results are not stored
+  const T* xr = x + (t < rows ? t : 0) * x_stride;
+  const T* wr = w + (int64_t)(n < N ? n : 0) * K;
+  const Frag zero = {};
+  f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int k0 = 32 * wv; k0 < K; k0 += 32 * PJ_WAVES) {
+    const bool in_k = k0 + 8 * lg < K;
+    const int k = in_k ? k0 + 8 * lg : 0;
+    const Frag av = *reinterpret_cast<const Frag*>(xr + k);
+    const Frag bv = *reinterpret_cast<const Frag*>(wr + k);
+    acc = Mfma<T>::run(in_k ? av : zero, bv, acc);
+  }
+  part[wv][lane] = acc;
+  __syncthreads();
+  if (wv != 0) return;
+#pragma unroll
+  for (int o = 1; o < PJ_WAVES; ++o) acc += part[o][lane];
+  if (n >= N) return;
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    const int64_t row = (int64_t)blockIdx.x * 16 + 4 * lg + r;
+    if (row < rows) out[row * N + n] = acc[r];
+  }
+}
+
+// The same for widths that are no multiple of 8: one wave per result.
+template <typename T>
+__global__ __launch_bounds__(256) void project_f32_kernel(float* __restrict__ out, const T* __restrict__ x, int64_t x_stride,
+                                                          const T* __restrict__ w, int64_t rows, int N, int K) {
+  const int lane = threadIdx.x & 63;
+  const int64_t idx = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (idx >= rows * N) return;
+  const int64_t t = idx / N;
+  const int n = (int)(idx - t * N);
+  float acc = 0.f;
+  for (int k = lane; k < K; k += 64) acc = fmaf(to_f32(x[t * x_stride + k]), to_f32(w[(int64_t)n * K + k]), acc);
+  acc = wave_sum(acc);
+  if (lane == 0) out[idx] = acc;
+}
+
+// out[p][i] = g sigmoid(alpha g) (u + 1) with g = min(c a[p][i], limit), u = clamp(c a[p][ff + i], -limit, limit): a gated unit on
+// [gate | up] rows.  The rows are p = rows[j] (a token's sorted expert rows) for j < pairs, or j itself; c = coef[j], or 1: the
+// factor belongs on the layer's input, which it commutes with as the projections have no bias.
+template <typename T, bool VEC>
+__global__ void clamped_glu_kernel(T* __restrict__ out, const T* __restrict__ a, int64_t a_stride, const int32_t* __restrict__ rows,
+                                   const float* __restrict__ coef, int ff, float limit, float alpha) {
+  constexpr int W = VEC ? 8 : 1;
+  const int64_t j = blockIdx.x;
+  const int64_t p = rows != nullptr ? rows[j] : j;
+  const float c = coef != nullptr ? coef[j] : 1.f;
+  const T* row = a + p * a_stride;
+  for (int i = W * (blockIdx.y * blockDim.x + threadIdx.x); i < ff; i += W * gridDim.y * blockDim.x) {
+    const Vec<T, W> gv = ldvec<T, W>(row + i), uv = ldvec<T, W>(row + ff + i);
+    Vec<T, W> o;
+#pragma unroll
+    for (int k = 0; k < W; ++k) {
+      const float g = fminf(c * to_f32(gv.v[k]), limit);
+      const float u = fminf(fmaxf(c * to_f32(uv.v[k]), -limit), limit);
+      o.v[k] = from_f32<T>(g / (1.0f + expf(-alpha * g)) * (u + 1.0f));
+    }
+    stvec<T, W>(out + p * ff + i, o);
+  }
+}
+
 template <typename T>
 int launch_grouped(void* out, const void* in, int64_t in_stride, const void* w, const int32_t* src_row, const int32_t* tile_expert,
                    const int32_t* n_tiles, int gather, int gelu, int N, int K, int64_t max_tiles, bool mfma, int block,
@@ -477,7 +555,14 @@ int mi355_moe_route_grouped(int32_t* ids, float* weights, const float* logits, c
 int mi355_moe_route_scores(int32_t* ids, float* weights, const float* logits, const float* correction, int64_t tokens,
                            int num_experts, int top, int n_groups, int keep_groups, float scale, int score_fn, int group_best,
                            int renorm, void* stream) {
-  MI355_REQUIRE(ids && weights && logits, MI355_ERR_INVALID, "moe_route_grouped: null pointer");
+  return mi355_moe_route_scores_strided(ids, weights, logits, num_experts, correction, tokens, num_experts, top, n_groups, keep_groups,
+                                        scale, score_fn, group_best, renorm, stream);
+}
+
+int mi355_moe_route_scores_strided(int32_t* ids, float* weights, const float* logits, int64_t logit_stride, const float* correction,
+                                   int64_t tokens, int num_experts, int top, int n_groups, int keep_groups, float scale, int score_fn,
+                                   int group_best, int renorm, void* stream) {
+  MI355_REQUIRE(ids && weights && logits && logit_stride >= num_experts, MI355_ERR_INVALID, "moe_route_grouped: null pointer or short rows");
   MI355_REQUIRE((score_fn == 0 || score_fn == 1) && (group_best == 1 || group_best == 2), MI355_ERR_INVALID,
                 "moe_route_grouped: scores are sigmoid (0) or softmax (1), a group counts its best 1 or 2");
   MI355_REQUIRE(tokens >= 0 && num_experts > 0 && n_groups > 0 && num_experts % n_groups == 0 && keep_groups >= 1 &&
@@ -487,7 +572,7 @@ int mi355_moe_route_scores(int32_t* ids, float* weights, const float* logits, co
   if (tokens == 0) return MI355_OK;
   const size_t lds = (size_t)4 * (2 * num_experts + n_groups) * sizeof(float);
   hipLaunchKernelGGL(moe_route_grouped_kernel, dim3((unsigned)((tokens + 3) / 4)), dim3(256), lds, (hipStream_t)stream, ids,
-                     weights, logits, correction, tokens, num_experts, top, n_groups, keep_groups, scale, score_fn, group_best, renorm);
+                     weights, logits, logit_stride, correction, tokens, num_experts, top, n_groups, keep_groups, scale, score_fn, group_best, renorm);
   MI355_CHECK_LAUNCH("moe_route_grouped");
   return MI355_OK;
 }
@@ -544,5 +629,52 @@ int mi355_moe_grouped_linear(void* out, const void* in, int64_t in_stride, const
   });
   if (rc != MI355_OK) return rc;
   MI355_CHECK_LAUNCH("moe_grouped_linear");
+  return MI355_OK;
+}
+
+int mi355_project_f32(float* out, const void* x, int64_t x_stride, const void* weight, int64_t rows, int n, int k, int dtype, void* stream) {
+  MI355_REQUIRE(out && x && weight, MI355_ERR_INVALID, "project_f32: null pointer");
+  MI355_REQUIRE(rows >= 0 && rows < (1ll << 31) && n > 0 && n <= 65536 && k > 0 && x_stride >= k, MI355_ERR_INVALID, "project_f32: bad shape");
+  MI355_REQUIRE(dtype == MI355_BF16 || dtype == MI355_F16, MI355_ERR_UNSUPPORTED, "project_f32: 16-bit operands");
+  if (rows == 0) return MI355_OK;
+  const bool mfma = k % 8 == 0 && x_stride % 8 == 0 && aligned16(x) && aligned16(weight);
+  const dim3 grid((unsigned)cdiv(rows, 16), (unsigned)cdiv(n, 16));
+  const int64_t waves = rows * n;
+  MI355_REQUIRE(mfma || waves / 4 < (1ll << 31) - 1, MI355_ERR_UNSUPPORTED, "project_f32: too many results");
+#define MI355_PJ(T)                                                                                                                   \
+  do {                                                                                                                                \
+    if (mfma)                                                                                                                         \
+      hipLaunchKernelGGL((project_f32_mfma_kernel<T>), grid, dim3(64 * PJ_WAVES), 0, (hipStream_t)stream, out, (const T*)x, x_stride, \
+                         (const T*)weight, rows, n, k);                                                                               \
+    else                                                                                                                              \
+      hipLaunchKernelGGL((project_f32_kernel<T>), dim3((unsigned)((waves + 3) / 4)), dim3(256), 0, (hipStream_t)stream, out,          \
+                         (const T*)x, x_stride, (const T*)weight, rows, n, k);                                                        \
+  } while (0)
+  if (dtype == MI355_BF16) MI355_PJ(bf16_t);
+  else MI355_PJ(f16_t);
+#undef MI355_PJ
+  MI355_CHECK_LAUNCH("project_f32");
+  return MI355_OK;
+}
+
+int mi355_clamped_glu(void* out, const void* a, int64_t a_stride, const int32_t* rows, const float* coef, int64_t pairs, int ff,
+                      float limit, float alpha, int dtype, void* stream) {
+  MI355_REQUIRE(out && a, MI355_ERR_INVALID, "clamped_glu: null pointer");
+  MI355_REQUIRE(pairs >= 0 && pairs < (1ll << 31) && ff > 0 && a_stride >= 2 * (int64_t)ff && limit >= 0.f, MI355_ERR_INVALID,
+                "clamped_glu: bad shape");
+  if (pairs == 0) return MI355_OK;
+  const bool vec = dtype != MI355_F32 && ff % 8 == 0 && a_stride % 8 == 0 && aligned16(out) && aligned16(a);
+  const int per = cdiv(ff, vec ? 8 : 1);
+  const int threads = std::min(256, cdiv(per, 64) * 64);
+  const dim3 grid((unsigned)pairs, (unsigned)std::min(cdiv(per, threads), 64));
+  MI355_DISPATCH_DTYPE(dtype, "clamped_glu", {
+    if (vec)
+      hipLaunchKernelGGL((clamped_glu_kernel<T, true>), grid, dim3(threads), 0, (hipStream_t)stream, (T*)out, (const T*)a, a_stride, rows,
+                         coef, ff, limit, alpha);
+    else
+      hipLaunchKernelGGL((clamped_glu_kernel<T, false>), grid, dim3(threads), 0, (hipStream_t)stream, (T*)out, (const T*)a, a_stride, rows,
+                         coef, ff, limit, alpha);
+  });
+  MI355_CHECK_LAUNCH("clamped_glu");
   return MI355_OK;
 }

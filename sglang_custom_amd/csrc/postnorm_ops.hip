@@ -340,12 +340,13 @@ __global__ __launch_bounds__(256) void gated_group_rmsnorm_kernel(T* __restrict_
   }
 }
 
-// One wave per (token, head): out = o / rms(o) (* w) * silu(gate), or * sigmoid(gate) with gate_act 1
+// One wave per (token, head): out = o / rms(o) (* w) * silu(gate), or * sigmoid(gate) with gate_act 1; w [dv] shared by the heads,
+// or (w_per_head) [heads, dv]
 template <typename T>
 __global__ __launch_bounds__(256) void head_rmsnorm_gate_kernel(T* __restrict__ out, const float* __restrict__ o,
                                                                 const T* __restrict__ w, const T* __restrict__ gate,
                                                                 int64_t gate_stride, int64_t tokens, int heads, int dv, float eps,
-                                                                int gate_act) {
+                                                                int gate_act, int w_per_head) {
   const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
   const int64_t idx = (int64_t)blockIdx.x * 4 + wv;
   if (idx >= tokens * heads) return;
@@ -356,6 +357,7 @@ __global__ __launch_bounds__(256) void head_rmsnorm_gate_kernel(T* __restrict__ 
   for (int i = lane; i < dv; i += 64) q += r[i] * r[i];
   q = wave_sum(q);
   const float inv = 1.0f / sqrtf(q / (float)dv + eps);
+  if (w_per_head) w += (int64_t)h * dv;
   const T* g = gate + t * gate_stride + (int64_t)h * dv;
   T* dst = out + idx * dv;
   for (int i = lane; i < dv; i += 64) {
@@ -609,7 +611,12 @@ int mi355_head_rmsnorm_gate(void* out, const float* o, const void* weight, const
 
 int mi355_head_rmsnorm_gate_act(void* out, const float* o, const void* weight, const void* gate, int64_t gate_stride, int64_t tokens,
                                 int heads, int value_dim, float eps, int gate_act, int dtype, void* stream) {
-  MI355_REQUIRE(out && o && gate, MI355_ERR_INVALID, "head_rmsnorm_gate: null pointer");
+  return mi355_head_rmsnorm_gate_wide(out, o, weight, 0, gate, gate_stride, tokens, heads, value_dim, eps, gate_act, dtype, stream);
+}
+
+int mi355_head_rmsnorm_gate_wide(void* out, const float* o, const void* weight, int weight_per_head, const void* gate, int64_t gate_stride,
+                                 int64_t tokens, int heads, int value_dim, float eps, int gate_act, int dtype, void* stream) {
+  MI355_REQUIRE(out && o && gate && (weight || !weight_per_head), MI355_ERR_INVALID, "head_rmsnorm_gate: null pointer");
   MI355_REQUIRE(gate_act == 0 || gate_act == 1, MI355_ERR_INVALID, "head_rmsnorm_gate: the gate is silu (0) or sigmoid (1)");
   MI355_REQUIRE(tokens >= 0 && heads > 0 && value_dim > 0 && gate_stride >= (int64_t)heads * value_dim, MI355_ERR_INVALID,
                 "head_rmsnorm_gate: bad shape");
@@ -617,7 +624,7 @@ int mi355_head_rmsnorm_gate_act(void* out, const float* o, const void* weight, c
   const unsigned grid = (unsigned)((tokens * heads + 3) / 4);
   MI355_DISPATCH_DTYPE(dtype, "head_rmsnorm_gate", {
     hipLaunchKernelGGL((head_rmsnorm_gate_kernel<T>), dim3(grid), dim3(256), 0, (hipStream_t)stream, (T*)out, o, (const T*)weight,
-                       (const T*)gate, gate_stride, tokens, heads, value_dim, eps, gate_act);
+                       (const T*)gate, gate_stride, tokens, heads, value_dim, eps, gate_act, weight_per_head);
   });
   MI355_CHECK_LAUNCH("head_rmsnorm_gate");
   return MI355_OK;

@@ -284,6 +284,172 @@ int launch_delta(float* out, float* state, const void* q, const void* k, const v
   return MI355_OK;
 }
 
+// Matrix memory with exponential gates.  Per head and token, from two fp32 logits: the log input gate
+// i = cap tanh((zi + bi) / cap), the log forget gate f = logsigmoid(cap tanh((zf + bf) / cap)), and
+//     m' = max(f + m, i);   S <- e^(f + m - m') S + e^(i - m') k v^T;   n <- e^(f + m - m') n + e^(i - m') k;   m <- m'
+//     o = S^T q / (max(|n . q|, e^-m) + 1e-6)            (q times q_scale; S, n and m start at zero)
+// Same layout as above for S.  The normaliser n is one more column of S whose value is always 1: a fifth wave carries it
+// (64 lanes share its dk channels) beside the four that carry the block's 32 columns, and the division happens when a stage's
+// read-outs leave LDS in whole rows.  Every block of value columns keeps a copy of (n, m) of its own in norm_state
+// [slots, heads, blocks, dk + 1] (m last): a block that starts late must not find what another one has already advanced.
+constexpr int MM_THREADS = 320;
+
+template <typename VT, int R>
+__global__ __launch_bounds__(MM_THREADS) void matrix_memory_kernel(
+    float* __restrict__ out, float* __restrict__ state, float* __restrict__ norm_state, const VT* __restrict__ q,
+    const VT* __restrict__ k, const VT* __restrict__ v, const float* __restrict__ in_logits, const float* __restrict__ forget_logits,
+    const float* __restrict__ in_bias, const float* __restrict__ forget_bias, const int32_t* __restrict__ req_to_state,
+    const int64_t* __restrict__ req_pool_indices, const int32_t* __restrict__ seg_start, const int32_t* __restrict__ seg_len,
+    const int64_t* __restrict__ positions, int heads, int dk, int dv, int64_t q_token_stride, int64_t k_token_stride,
+    int64_t v_token_stride, int64_t gate_token_stride, float q_scale, float cap) {
+  constexpr int DKP = R * RC_RG;
+  constexpr int RN = DKP > 64 ? DKP / 64 : 1;       // channels of n per lane of the fifth wave
+  __shared__ __attribute__((aligned(16))) float qs[RC_TC][DKP];
+  __shared__ __attribute__((aligned(16))) float ks[RC_TC][DKP];
+  __shared__ float vs[RC_TC][RC_COLS];
+  __shared__ float os[RC_TC][RC_COLS + 1];
+  __shared__ float li[RC_TC], lf[RC_TC], keep[RC_TC], write[RC_TC], floor_[RC_TC], inv_den[RC_TC];
+  __shared__ float m_sh[2];
+  const int b = blockIdx.z, h = blockIdx.y, c0 = blockIdx.x * RC_COLS;
+  const int tid = threadIdx.x;
+  const int rg = tid & (RC_RG - 1), cl = tid >> 3;
+  const int col = c0 + cl;
+  const bool column_wave = tid < 256;
+  const int nl = tid & 63;
+  const int64_t t0 = seg_start != nullptr ? seg_start[b] : b;
+  const int n_tok = seg_len != nullptr ? seg_len[b] : 1;
+  if (n_tok <= 0) return;
+  const int64_t slot = req_to_state[req_pool_indices[b]];
+  float* sp = state + ((slot * heads + h) * (int64_t)dk) * dv;
+  float* np = norm_state + ((slot * heads + h) * (int64_t)gridDim.x + blockIdx.x) * (dk + 1);
+  const bool fresh = positions[t0] == 0;
+  float S[R], nv[RN];
+  if (column_wave) {
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+      const int i = rg * R + r;
+      S[r] = (!fresh && i < dk && col < dv) ? sp[(int64_t)i * dv + col] : 0.f;
+    }
+  } else {
+#pragma unroll
+    for (int r = 0; r < RN; ++r) {
+      const int i = nl * RN + r;
+      nv[r] = (!fresh && i < dk) ? np[i] : 0.f;
+    }
+    if (nl == 0) m_sh[0] = fresh ? 0.f : np[dk];
+  }
+  const float bi = in_bias[h], bf = forget_bias[h];
+  int par = 0;
+  for (int base = 0; base < n_tok; base += RC_TC, par ^= 1) {
+    const int m = min(RC_TC, n_tok - base);
+    if (tid < m) {
+      const int64_t g = (t0 + base + tid) * gate_token_stride + h;
+      li[tid] = cap * tanhf((in_logits[g] + bi) / cap);
+      lf[tid] = log_sigmoid_f(cap * tanhf((forget_logits[g] + bf) / cap));
+    }
+    __syncthreads();
+    if (tid < m) {
+      // the running maximum up to this token, by the same operations in the same order wherever the step was cut
+      float prev = m_sh[par], cur = prev;
+      for (int j = 0; j <= tid; ++j) {
+        prev = cur;
+        cur = fmaxf(lf[j] + prev, li[j]);
+      }
+      keep[tid] = expf(lf[tid] + prev - cur);
+      write[tid] = expf(li[tid] - cur);
+      floor_[tid] = expf(-cur);
+      if (tid == m - 1) m_sh[par ^ 1] = cur;
+    }
+    for (int e = tid; e < m * RC_COLS; e += MM_THREADS) {
+      const int tt = e / RC_COLS, c = e - tt * RC_COLS;
+      vs[tt][c] = (c0 + c < dv) ? to_f32(v[(t0 + base + tt) * v_token_stride + (int64_t)h * dv + c0 + c]) : 0.f;
+    }
+    for (int e = tid; e < m * DKP; e += MM_THREADS) {
+      const int tt = e / DKP, i = e - tt * DKP;
+      const int64_t t = t0 + base + tt;
+      qs[tt][i] = i < dk ? to_f32(q[t * q_token_stride + (int64_t)h * dk + i]) * q_scale : 0.f;
+      ks[tt][i] = i < dk ? to_f32(k[t * k_token_stride + (int64_t)h * dk + i]) : 0.f;
+    }
+    __syncthreads();
+    if (column_wave) {
+      for (int tt = 0; tt < m; ++tt) {
+        const float wv = write[tt] * vs[tt][cl], a = keep[tt];
+        float acc = 0.f;
+#pragma unroll
+        for (int r4 = 0; r4 < R; r4 += 4) {
+          const float4 k4 = *reinterpret_cast<const float4*>(&ks[tt][rg * R + r4]);
+          const float4 q4 = *reinterpret_cast<const float4*>(&qs[tt][rg * R + r4]);
+          S[r4 + 0] = fmaf(a, S[r4 + 0], k4.x * wv);
+          S[r4 + 1] = fmaf(a, S[r4 + 1], k4.y * wv);
+          S[r4 + 2] = fmaf(a, S[r4 + 2], k4.z * wv);
+          S[r4 + 3] = fmaf(a, S[r4 + 3], k4.w * wv);
+          acc = fmaf(S[r4 + 0], q4.x, acc);
+          acc = fmaf(S[r4 + 1], q4.y, acc);
+          acc = fmaf(S[r4 + 2], q4.z, acc);
+          acc = fmaf(S[r4 + 3], q4.w, acc);
+        }
+        acc += __shfl_xor(acc, 1, 64);
+        acc += __shfl_xor(acc, 2, 64);
+        acc += __shfl_xor(acc, 4, 64);
+        if (rg == 0) os[tt][cl] = acc;
+      }
+    } else {
+      for (int tt = 0; tt < m; ++tt) {
+        const float a = keep[tt], w = write[tt];
+        float dot = 0.f;
+#pragma unroll
+        for (int r = 0; r < RN; ++r) {
+          const int i = nl * RN + r;
+          if (DKP >= 64 || i < DKP) {
+            nv[r] = fmaf(a, nv[r], ks[tt][i] * w);
+            dot = fmaf(nv[r], qs[tt][i], dot);
+          }
+        }
+        dot = wave_sum(dot);
+        if (nl == 0) inv_den[tt] = 1.0f / (fmaxf(fabsf(dot), floor_[tt]) + 1e-6f);
+      }
+    }
+    __syncthreads();
+    for (int e = tid; e < m * RC_COLS; e += MM_THREADS) {
+      const int tt = e / RC_COLS, c = e - tt * RC_COLS;
+      if (c0 + c < dv) out[((t0 + base + tt) * heads + h) * (int64_t)dv + c0 + c] = os[tt][c] * inv_den[tt];
+    }
+  }
+  if (column_wave) {
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+      const int i = rg * R + r;
+      if (i < dk && col < dv) sp[(int64_t)i * dv + col] = S[r];
+    }
+  } else {
+#pragma unroll
+    for (int r = 0; r < RN; ++r) {
+      const int i = nl * RN + r;
+      if (i < dk) np[i] = nv[r];
+    }
+    if (nl == 0) np[dk] = m_sh[par];
+  }
+}
+
+template <typename VT>
+int launch_matrix_memory(float* out, float* state, float* norm_state, const void* q, const void* k, const void* v,
+                         const float* in_logits, const float* forget_logits, const float* in_bias, const float* forget_bias,
+                         const int32_t* req_to_state, const int64_t* req_pool_indices, const int32_t* seg_start, const int32_t* seg_len,
+                         const int64_t* positions, int64_t batch, int heads, int dk, int dv, int64_t qs, int64_t ks, int64_t vs,
+                         int64_t gs, float q_scale, float cap, hipStream_t stream) {
+  const dim3 grid((unsigned)cdiv(dv, RC_COLS), (unsigned)heads, (unsigned)batch);
+#define MI355_MM_LAUNCH(R)                                                                                                       \
+  hipLaunchKernelGGL((matrix_memory_kernel<VT, R>), grid, dim3(MM_THREADS), 0, stream, out, state, norm_state, (const VT*)q,     \
+                     (const VT*)k, (const VT*)v, in_logits, forget_logits, in_bias, forget_bias, req_to_state, req_pool_indices, \
+                     seg_start, seg_len, positions, heads, dk, dv, qs, ks, vs, gs, q_scale, cap)
+  if (dk <= 32) MI355_MM_LAUNCH(4);
+  else if (dk <= 64) MI355_MM_LAUNCH(8);
+  else if (dk <= 128) MI355_MM_LAUNCH(16);
+  else MI355_MM_LAUNCH(32);
+#undef MI355_MM_LAUNCH
+  return MI355_OK;
+}
+
 }  // namespace
 }  // namespace mi355
 
@@ -386,5 +552,33 @@ int mi355_gated_delta_rule_ex(float* out, float* state, const void* q, const voi
   });
   if (rc != MI355_OK) return rc;
   MI355_CHECK_LAUNCH("gated_delta_rule");
+  return MI355_OK;
+}
+
+int mi355_matrix_memory_value_block(void) { return RC_COLS; }
+
+int mi355_matrix_memory(float* out, float* state, float* norm_state, const void* q, const void* k, const void* v,
+                        const float* in_logits, const float* forget_logits, const float* in_bias, const float* forget_bias,
+                        const int32_t* req_to_state, const int64_t* req_pool_indices, const int32_t* seg_start, const int32_t* seg_len,
+                        const int64_t* positions, int64_t batch, int heads, int key_dim, int value_dim, int norm_blocks,
+                        int64_t q_token_stride, int64_t k_token_stride, int64_t v_token_stride, int64_t gate_token_stride,
+                        float q_scale, float gate_cap, int dtype, void* stream) {
+  MI355_REQUIRE(out && state && norm_state && q && k && v && in_logits && forget_logits && in_bias && forget_bias && req_to_state &&
+                    req_pool_indices && positions, MI355_ERR_INVALID, "matrix_memory: null pointer");
+  MI355_REQUIRE((seg_start == nullptr) == (seg_len == nullptr), MI355_ERR_INVALID, "matrix_memory: seg_start and seg_len come together");
+  MI355_REQUIRE(batch >= 0 && batch <= 65535 && heads > 0 && heads <= 65535 && key_dim > 0 && value_dim > 0 && gate_cap > 0.f &&
+                    gate_token_stride >= heads, MI355_ERR_INVALID, "matrix_memory: bad shape");
+  MI355_REQUIRE(norm_blocks == cdiv(value_dim, RC_COLS), MI355_ERR_INVALID,
+                "matrix_memory: %d copies of the normaliser for %d value columns (one per %d)", norm_blocks, value_dim, RC_COLS);
+  MI355_REQUIRE(key_dim <= 256, MI355_ERR_UNSUPPORTED, "matrix_memory: key width %d above 256", key_dim);
+  if (batch == 0) return MI355_OK;
+  int rc = MI355_OK;
+  MI355_DISPATCH_DTYPE(dtype, "matrix_memory", {
+    rc = launch_matrix_memory<T>(out, state, norm_state, q, k, v, in_logits, forget_logits, in_bias, forget_bias, req_to_state,
+                                 req_pool_indices, seg_start, seg_len, positions, batch, heads, key_dim, value_dim, q_token_stride,
+                                 k_token_stride, v_token_stride, gate_token_stride, q_scale, gate_cap, (hipStream_t)stream);
+  });
+  if (rc != MI355_OK) return rc;
+  MI355_CHECK_LAUNCH("matrix_memory");
   return MI355_OK;
 }

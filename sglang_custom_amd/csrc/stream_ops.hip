@@ -1,6 +1,8 @@
 // Kernels around a 32-bit residual stream whose sequences carry state from step to step:
 //   * token + hashed-bigram embedding (the previous token of a sequence is state),
 //   * weight-only layer norm fused with the token shift (the previous token's normed row is state),
+//   * the layer norm of a sublayer's output, its sum into the stream and the layer norm in front of the next sublayer as one
+//     launch,
 //   * the commit of a step's new state rows,
 //   * tanh-GELU-and-mul, and the sigmoid-gated residual update.
 // Every reduction, normalisation, gate and the residual sum run in fp32 whatever the activation dtype T is;
@@ -125,6 +127,174 @@ __global__ __launch_bounds__(256) void layernorm_shift_kernel(
     }
     stvec<T, W>(h_out + t * D + i, ho);
     stvec<T, W>(hs_out + t * D + i, so);
+  }
+}
+
+// One workgroup per token:  x[t] += LN(b) * w_out,  h[t] = LN(x[t]) * w_next  (w_next null: no h), with
+// b = sum_j y[rows[t][j]] (rows null: y[t]) + sigmoid(gate[t]) * y2[t] (y2 null: nothing).  KEEP > 0: the row stays in
+// registers, KEEP groups of eight features per thread (D <= 2048 KEEP, 16-byte accesses); KEEP 0: any D, the row in LDS.
+struct LnAddParams {
+  float* x;
+  void* h;
+  const void* y;
+  const int32_t* rows;
+  const void* y2;
+  const float* gate;
+  const void* w_out;
+  const void* w_next;
+  int64_t y_stride, y2_stride, gate_stride, D;
+  int n_rows;
+  float eps;
+};
+
+template <typename T> __device__ __forceinline__ void ld8f(const T* p, float* o) {
+  if constexpr (sizeof(T) == 2) {
+    const Vec<T, 8> v = ldvec<T, 8>(p);
+#pragma unroll
+    for (int k = 0; k < 8; ++k) o[k] = to_f32(v.v[k]);
+  } else {
+    const Vec<T, 4> a = ldvec<T, 4>(p), b = ldvec<T, 4>(p + 4);
+#pragma unroll
+    for (int k = 0; k < 4; ++k) { o[k] = to_f32(a.v[k]); o[4 + k] = to_f32(b.v[k]); }
+  }
+}
+template <typename T> __device__ __forceinline__ void st8f(T* p, const float* o) {
+  if constexpr (sizeof(T) == 2) {
+    Vec<T, 8> v;
+#pragma unroll
+    for (int k = 0; k < 8; ++k) v.v[k] = from_f32<T>(o[k]);
+    stvec<T, 8>(p, v);
+  } else {
+    Vec<T, 4> a, b;
+#pragma unroll
+    for (int k = 0; k < 4; ++k) { a.v[k] = from_f32<T>(o[k]); b.v[k] = from_f32<T>(o[4 + k]); }
+    stvec<T, 4>(p, a);
+    stvec<T, 4>(p + 4, b);
+  }
+}
+
+// (v - mean) / sqrt(var + eps) of a row held as G groups of eight per thread (groups past D hold zeros)
+template <int G>
+__device__ __forceinline__ void ln_regs(float (&v)[G][8], int64_t D, float eps, float* red) {
+  float s = 0.f;
+#pragma unroll
+  for (int g = 0; g < G; ++g)
+#pragma unroll
+    for (int k = 0; k < 8; ++k) s += v[g][k];
+  const float mean = block_sum(s, red) / (float)D;
+  float q = 0.f;
+#pragma unroll
+  for (int g = 0; g < G; ++g) {
+    const bool live = 8 * ((int64_t)threadIdx.x + 256 * g) < D;
+#pragma unroll
+    for (int k = 0; k < 8; ++k) {
+      const float d = live ? v[g][k] - mean : 0.f;
+      v[g][k] = d;
+      q += d * d;
+    }
+  }
+  const float inv = 1.0f / sqrtf(block_sum(q, red) / (float)D + eps);
+#pragma unroll
+  for (int g = 0; g < G; ++g)
+#pragma unroll
+    for (int k = 0; k < 8; ++k) v[g][k] *= inv;
+}
+
+// the same of a row in LDS, in place; every thread touches the same elements in all passes
+__device__ __forceinline__ void ln_lds(float* buf, int64_t D, float eps, float* red) {
+  float s = 0.f;
+  for (int64_t i = threadIdx.x; i < D; i += 256) s += buf[i];
+  const float mean = block_sum(s, red) / (float)D;
+  float q = 0.f;
+  for (int64_t i = threadIdx.x; i < D; i += 256) {
+    const float d = buf[i] - mean;
+    q += d * d;
+  }
+  const float inv = 1.0f / sqrtf(block_sum(q, red) / (float)D + eps);
+  for (int64_t i = threadIdx.x; i < D; i += 256) buf[i] = (buf[i] - mean) * inv;
+}
+
+template <typename T, int KEEP>
+__global__ __launch_bounds__(256) void layernorm_residual_add_kernel(const LnAddParams p) {
+  __shared__ float red[16];
+  const int64_t t = blockIdx.x, D = p.D;
+  float* xr = p.x + t * D;
+  const T* y = static_cast<const T*>(p.y);
+  const T* y2 = static_cast<const T*>(p.y2);
+  const T* w_out = static_cast<const T*>(p.w_out);
+  const T* w_next = static_cast<const T*>(p.w_next);
+  T* h = static_cast<T*>(p.h) + t * D;
+  const float sg = y2 != nullptr ? 1.0f / (1.0f + expf(-p.gate[t * p.gate_stride])) : 0.f;
+  if constexpr (KEEP > 0) {
+    float v[KEEP][8];
+#pragma unroll
+    for (int g = 0; g < KEEP; ++g) {
+      const int64_t i = 8 * ((int64_t)threadIdx.x + 256 * g);
+#pragma unroll
+      for (int k = 0; k < 8; ++k) v[g][k] = 0.f;
+      if (i >= D) continue;
+      if (p.rows == nullptr) {
+        ld8f<T>(y + t * p.y_stride + i, v[g]);
+      } else {
+        for (int j = 0; j < p.n_rows; ++j) {      // fixed order: the sum does not depend on where the rows lie
+          float e[8];
+          ld8f<T>(y + (int64_t)p.rows[t * p.n_rows + j] * p.y_stride + i, e);
+#pragma unroll
+          for (int k = 0; k < 8; ++k) v[g][k] += e[k];
+        }
+      }
+      if (y2 != nullptr) {
+        float e[8];
+        ld8f<T>(y2 + t * p.y2_stride + i, e);
+#pragma unroll
+        for (int k = 0; k < 8; ++k) v[g][k] += sg * e[k];
+      }
+    }
+    ln_regs<KEEP>(v, D, p.eps, red);
+#pragma unroll
+    for (int g = 0; g < KEEP; ++g) {
+      const int64_t i = 8 * ((int64_t)threadIdx.x + 256 * g);
+      if (i >= D) continue;
+      float w[8], r[8];
+      ld8f<T>(w_out + i, w);
+      ld8f<float>(xr + i, r);
+#pragma unroll
+      for (int k = 0; k < 8; ++k) v[g][k] = r[k] + v[g][k] * w[k];
+      st8f<float>(xr + i, v[g]);
+    }
+    if (w_next == nullptr) return;
+    ln_regs<KEEP>(v, D, p.eps, red);
+#pragma unroll
+    for (int g = 0; g < KEEP; ++g) {
+      const int64_t i = 8 * ((int64_t)threadIdx.x + 256 * g);
+      if (i >= D) continue;
+      float w[8];
+      ld8f<T>(w_next + i, w);
+#pragma unroll
+      for (int k = 0; k < 8; ++k) w[k] *= v[g][k];
+      st8f<T>(h + i, w);
+    }
+  } else {
+    extern __shared__ __attribute__((aligned(16))) float sm[];      // [D]; a thread touches the same elements in every pass
+    for (int64_t i = threadIdx.x; i < D; i += 256) {
+      float b = 0.f;
+      if (p.rows == nullptr) {
+        b = to_f32(y[t * p.y_stride + i]);
+      } else {
+        for (int j = 0; j < p.n_rows; ++j) b += to_f32(y[(int64_t)p.rows[t * p.n_rows + j] * p.y_stride + i]);
+      }
+      if (y2 != nullptr) b += sg * to_f32(y2[t * p.y2_stride + i]);
+      sm[i] = b;
+    }
+    ln_lds(sm, D, p.eps, red);
+    for (int64_t i = threadIdx.x; i < D; i += 256) {
+      const float r = xr[i] + sm[i] * to_f32(w_out[i]);
+      xr[i] = r;
+      sm[i] = r;
+    }
+    if (w_next == nullptr) return;
+    ln_lds(sm, D, p.eps, red);
+    for (int64_t i = threadIdx.x; i < D; i += 256) h[i] = from_f32<T>(sm[i] * to_f32(w_next[i]));
   }
 }
 
@@ -316,5 +486,38 @@ int mi355_gated_residual_add(float* x, const void* g1, const void* b1, const voi
                        (const T*)y1, (const T*)g2, (const T*)b2, (const T*)y2, rows, d, g_stride, y1_stride, y2_stride);
   });
   MI355_CHECK_LAUNCH("gated_residual_add");
+  return MI355_OK;
+}
+
+int mi355_layernorm_residual_add(float* x, void* h, const void* y, int64_t y_stride, const int32_t* rows, int n_rows, const void* y2,
+                                 int64_t y2_stride, const float* y2_gate, int64_t gate_stride, const void* w_out, const void* w_next,
+                                 int64_t tokens, int64_t hidden, float eps, int dtype, void* stream) {
+  MI355_REQUIRE(x && y && w_out && (h == nullptr) == (w_next == nullptr), MI355_ERR_INVALID, "layernorm_residual_add: null pointer");
+  MI355_REQUIRE((y2 == nullptr) == (y2_gate == nullptr) && (rows == nullptr || n_rows > 0), MI355_ERR_INVALID,
+                "layernorm_residual_add: the second branch comes with its gate, picked rows with their count");
+  MI355_REQUIRE(tokens >= 0 && tokens < (1ll << 31) && hidden > 0 && hidden <= 32768 && y_stride >= hidden &&
+                    (y2 == nullptr || y2_stride >= hidden), MI355_ERR_INVALID, "layernorm_residual_add: bad shape");
+  if (tokens == 0) return MI355_OK;
+  LnAddParams p;
+  p.x = x; p.h = h; p.y = y; p.rows = rows; p.y2 = y2; p.gate = y2_gate; p.w_out = w_out; p.w_next = w_next;
+  p.y_stride = y_stride; p.y2_stride = y2_stride; p.gate_stride = gate_stride; p.D = hidden; p.n_rows = n_rows; p.eps = eps;
+  const bool vec = hidden % 8 == 0 && hidden <= 8192 && y_stride % 8 == 0 && aligned16(x) && aligned16(y) && aligned16(w_out) &&
+                   (h == nullptr || (aligned16(h) && aligned16(w_next))) && (y2 == nullptr || (aligned16(y2) && y2_stride % 8 == 0));
+  const dim3 grid((unsigned)tokens), block(256);
+  MI355_DISPATCH_DTYPE(dtype, "layernorm_residual_add", {
+    if (vec && hidden <= 2048) {
+      hipLaunchKernelGGL((layernorm_residual_add_kernel<T, 1>), grid, block, 0, (hipStream_t)stream, p);
+    } else if (vec && hidden <= 4096) {
+      hipLaunchKernelGGL((layernorm_residual_add_kernel<T, 2>), grid, block, 0, (hipStream_t)stream, p);
+    } else if (vec) {
+      hipLaunchKernelGGL((layernorm_residual_add_kernel<T, 4>), grid, block, 0, (hipStream_t)stream, p);
+    } else {
+      auto kern = layernorm_residual_add_kernel<T, 0>;
+      const size_t lds = (size_t)hidden * sizeof(float);
+      if (lds > 48 * 1024) (void)hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+      hipLaunchKernelGGL(kern, grid, block, lds, (hipStream_t)stream, p);
+    }
+  });
+  MI355_CHECK_LAUNCH("layernorm_residual_add");
   return MI355_OK;
 }

@@ -1207,6 +1207,23 @@ def latent_norms_rope_write(a: torch.Tensor, q_weight: torch.Tensor, kv_weight: 
     return cq
 
 
+def latent_rows_write(a: torch.Tensor, q_cols: int, kv_weight: torch.Tensor, positions: torch.Tensor, out_cache_loc: torch.Tensor,
+                      inv_freq: Optional[torch.Tensor], cache: torch.Tensor, rank: int, rope_dim: int, rot_dims: int, interleaved: bool,
+                      rot_mag: float, eps: float) -> None:
+    """a [T, >= q_cols + rank + rope_dim]: writes the cache rows [RMSnorm(kv latent) * kv_weight | rot(shared key part)] at
+    out_cache_loc; the first q_cols columns (queries without a norm) are not touched."""
+    _gpu(a, kv_weight, positions, out_cache_loc, inv_freq, cache)
+    assert a.dim() == 2 and a.stride(1) == 1 and cache.is_contiguous() and cache.dtype == a.dtype == kv_weight.dtype
+    assert a.shape[1] >= q_cols + rank + rope_dim and cache.shape[-1] == rank + rope_dim and kv_weight.numel() == rank
+    assert rot_dims == 0 or (inv_freq.dtype == torch.float32 and inv_freq.numel() >= rot_dims // 2)
+    assert positions.dtype == torch.int64 and out_cache_loc.dtype == torch.int64 and out_cache_loc.numel() == a.shape[0]
+    assert positions.is_contiguous() and out_cache_loc.is_contiguous()
+    check(_lib_().mi355_latent_rows_write(None, cache.data_ptr(), a.data_ptr(), None, kv_weight.data_ptr(), positions.data_ptr(),
+                                          out_cache_loc.data_ptr(), _p(inv_freq) if rot_dims else None, a.shape[0], a.stride(0),
+                                          int(q_cols), int(rank), int(rope_dim), int(rot_dims), int(bool(interleaved)), float(rot_mag),
+                                          cache.shape[0], float(eps), _dt(a), _stream(a)), "latent_rows_write")
+
+
 def latent_window_attention_block_tokens(heads: int, rank: int, rope_dim: int, dtype: torch.dtype) -> int:
     """Most consecutive tokens of one sequence that a workgroup of latent_window_attention takes (0: shape not served)."""
     return int(_lib_().mi355_latent_window_attention_block_tokens(heads, rank, rope_dim, _DT[dtype]))
@@ -1217,22 +1234,25 @@ def latent_window_attention_splits(tokens: int, heads: int, rank: int, window: i
     at least 128 keys each."""
     if dtype not in (torch.bfloat16, torch.float16) or rank > 512:
         return 1
-    keys = min(window, max_position + 1)
+    keys = min(window, max_position + 1) if window > 0 else max_position + 1
     wgs = max(1, tokens * ((heads + 63) // 64))
     return int(max(1, min(64, (512 + wgs - 1) // wgs, keys // 128)))
 
 
 def latent_window_attention(qa: torch.Tensor, qr: torch.Tensor, cache: torch.Tensor, out: torch.Tensor, req_to_token: torch.Tensor,
-                            req_pool_indices: torch.Tensor, positions: torch.Tensor, sink: torch.Tensor, inv_freq: torch.Tensor,
+                            req_pool_indices: torch.Tensor, positions: torch.Tensor, sink: Optional[torch.Tensor], inv_freq: torch.Tensor,
                             rot_dims: int, window: int, scale: float, gate: Optional[torch.Tensor] = None, tok_req=None,
-                            blocks=None, num_splits: int = 1) -> torch.Tensor:
+                            blocks=None, num_splits: int = 1, interleaved: bool = False, rot_mag: float = 1.0) -> torch.Tensor:
     """qa [T, H, rank] and out [T, H, rank] (any token / head strides), qr [T, H, rope_dim] unrotated, cache
-    [slots, rank + rope_dim], gate [T, H] logits (row-strided) or None, blocks int32 [n, 2] runs of tokens or None."""
+    [slots, rank + rope_dim], gate [T, H] logits (row-strided) or None, blocks int32 [n, 2] runs of tokens or None.
+    window 0: every earlier token; sink None: a plain softmax; the rotation of qr pairs feature i with i + rot_dims / 2, or
+    2 i with 2 i + 1 (interleaved), cos and sin times rot_mag."""
     _gpu(qa, qr, cache, out, req_to_token, req_pool_indices, positions, sink, inv_freq, gate, tok_req, blocks)
     T, H, rank = qa.shape
     rope_dim = cache.shape[-1] - rank
     assert out.shape == qa.shape and qa.stride(2) == 1 and out.stride(2) == 1 and cache.is_contiguous()
-    assert qa.dtype == out.dtype == cache.dtype and sink.dtype == torch.float32 and sink.numel() == H and sink.is_contiguous()
+    assert qa.dtype == out.dtype == cache.dtype
+    assert sink is None or (sink.dtype == torch.float32 and sink.numel() == H and sink.is_contiguous())
     assert req_to_token.dtype == torch.int32 and req_pool_indices.dtype == torch.int64 and positions.dtype == torch.int64
     if rope_dim:
         assert qr.shape == (T, H, rope_dim) and qr.stride(2) == 1 and qr.dtype == qa.dtype and inv_freq.dtype == torch.float32
@@ -1247,12 +1267,12 @@ def latent_window_attention(qa: torch.Tensor, qr: torch.Tensor, cache: torch.Ten
     if num_splits > 1:
         assert blocks is None, "key splits serve launches of one token per run"
         scratch = torch.empty(num_splits * T * H * (rank + 2), dtype=torch.float32, device=qa.device)
-    check(_lib_().mi355_latent_window_attention(
+    check(_lib_().mi355_latent_attention(
         out.data_ptr(), qa.data_ptr(), _p(qr) if rope_dim else None, cache.data_ptr(), _p(gate), req_to_token.data_ptr(),
-        req_pool_indices.data_ptr(), _p(tok_req), positions.data_ptr(), _p(blocks), nb, sink.data_ptr(), _p(inv_freq),
+        req_pool_indices.data_ptr(), _p(tok_req), positions.data_ptr(), _p(blocks), nb, _p(sink), _p(inv_freq) if rot_dims else None,
         qa.stride(0), qa.stride(1), qr.stride(0) if rope_dim else 0, qr.stride(1) if rope_dim else 0, out.stride(0), out.stride(1),
-        gate.stride(0) if gate is not None else 0, req_to_token.stride(0), H, rank, rope_dim, rot_dims, int(window), float(scale),
-        int(num_splits), _p(scratch), T, _dt(qa), _stream(qa)), "latent_window_attention")
+        gate.stride(0) if gate is not None else 0, req_to_token.stride(0), H, rank, rope_dim, rot_dims,
+        int(bool(interleaved)), float(rot_mag), int(window), float(scale), int(num_splits), _p(scratch), T, _dt(qa), _stream(qa)), "latent_window_attention")
     return out
 
 
@@ -1590,19 +1610,21 @@ def branch_residual_add(x: torch.Tensor, a: torch.Tensor, wa: Optional[torch.Ten
 
 def head_rmsnorm_gate_act(o: torch.Tensor, weight: Optional[torch.Tensor], gate: torch.Tensor, eps: float, out_dtype: torch.dtype,
                           gate_act: str = "silu") -> torch.Tensor:
-    """head_rmsnorm_gate with the gate's function chosen: "silu" or "sigmoid"."""
+    """head_rmsnorm_gate with the gate's function chosen ("silu" or "sigmoid") and the weight shared by the heads ([dv]) or one
+    per head ([H * dv])."""
     _gpu(o, weight, gate)
     T, H, dv = o.shape
     assert o.dtype == torch.float32 and o.is_contiguous() and gate.shape == (T, H * dv) and gate.stride(1) == 1
-    assert gate.dtype == out_dtype and (weight is None or (weight.dtype == out_dtype and weight.numel() == dv and weight.is_contiguous()))
+    assert gate.dtype == out_dtype and (weight is None or (weight.dtype == out_dtype and weight.numel() in (dv, H * dv) and weight.is_contiguous()))
+    per_head = weight is not None and H > 1 and weight.numel() == H * dv
     out = torch.empty((T, H * dv), dtype=out_dtype, device=o.device)
-    check(_lib_().mi355_head_rmsnorm_gate_act(out.data_ptr(), o.data_ptr(), _p(weight), gate.data_ptr(), gate.stride(0), T, H, dv,
-                                              float(eps), {"silu": 0, "sigmoid": 1}[gate_act], _dt(gate), _stream(o)),
+    check(_lib_().mi355_head_rmsnorm_gate_wide(out.data_ptr(), o.data_ptr(), _p(weight), int(per_head), gate.data_ptr(), gate.stride(0), T, H,
+                                               dv, float(eps), {"silu": 0, "sigmoid": 1}[gate_act], _dt(gate), _stream(o)),
           "head_rmsnorm_gate")
     return out
 
 
-ACTIVATIONS = {"none": 0, "silu": 1, "relu2": 2}
+ACTIVATIONS = {"none": 0, "silu": 1, "relu2": 2, "gelu_erf": 3}
 
 
 def causal_conv(u: torch.Tensor, w1: torch.Tensor, state: torch.Tensor, req_to_state: torch.Tensor, req_pool_indices: torch.Tensor,
@@ -1638,10 +1660,10 @@ def causal_conv(u: torch.Tensor, w1: torch.Tensor, state: torch.Tensor, req_to_s
 
 
 def activation(x: torch.Tensor, act: str) -> torch.Tensor:
-    """act(x) over a row-strided [T, d] block, contiguous result: "silu" or "relu2" (the square of relu)."""
+    """act(x) over a row-strided [T, d] block, contiguous result: "silu", "relu2" (the square of relu) or "gelu_erf"."""
     _gpu(x)
     T, d = x.shape
-    assert x.stride(1) == 1 and act in ("silu", "relu2")
+    assert x.stride(1) == 1 and act in ("silu", "relu2", "gelu_erf")
     out = torch.empty((T, d), dtype=x.dtype, device=x.device)
     check(_lib_().mi355_activation(out.data_ptr(), x.data_ptr(), x.stride(0), T, d, ACTIVATIONS[act], _dt(x), _stream(x)), "activation")
     return out
@@ -1765,11 +1787,108 @@ def moe_route_scores(logits: torch.Tensor, correction: Optional[torch.Tensor], t
     selection-only correction, a group scoring the sum of its group_best (1 or 2) best members, weights renormalised or not."""
     _gpu(logits, correction)
     T, E = logits.shape
-    assert logits.dtype == torch.float32 and logits.is_contiguous()
+    assert logits.dtype == torch.float32 and logits.stride(1) == 1
     assert correction is None or (correction.dtype == torch.float32 and correction.numel() == E)
     ids = torch.empty((T, top), dtype=torch.int32, device=logits.device)
     w = torch.empty((T, top), dtype=torch.float32, device=logits.device)
-    check(_lib_().mi355_moe_route_scores(ids.data_ptr(), w.data_ptr(), logits.data_ptr(), _p(correction), T, E, int(top), int(n_groups),
-                                         int(keep_groups), float(scale), {"sigmoid": 0, "softmax": 1}[score_fn], int(group_best),
-                                         int(bool(renorm)), _stream(logits)), "moe_route_scores")
+    check(_lib_().mi355_moe_route_scores_strided(ids.data_ptr(), w.data_ptr(), logits.data_ptr(), max(logits.stride(0), E), _p(correction), T,
+                                                 E, int(top), int(n_groups), int(keep_groups), float(scale),
+                                                 {"sigmoid": 0, "softmax": 1}[score_fn], int(group_best), int(bool(renorm)),
+                                                 _stream(logits)), "moe_route_scores")
     return ids, w
+
+
+# ------------------------------------------------------- layer norms around every sublayer, matrix memory, clamped experts
+def layernorm_residual_add(x: torch.Tensor, y: torch.Tensor, w_out: torch.Tensor, w_next: Optional[torch.Tensor], eps: float,
+                           rows: Optional[torch.Tensor] = None, y2: Optional[torch.Tensor] = None,
+                           y2_gate: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """x += LN(b) * w_out in place on the fp32 rows; returns LN(x) * w_next in the weights' dtype (None without w_next).
+    b = y [T, D], or with rows int32 [T, n] the sum of y[rows[t, j]], plus sigmoid(y2_gate [T], fp32, strided) * y2 [T, D]."""
+    _gpu(x, y, w_out, w_next, rows, y2, y2_gate)
+    assert x.dtype == torch.float32 and x.dim() == 2 and x.is_contiguous()
+    T, D = x.shape
+    assert y.dim() == 2 and y.shape[1] == D and y.stride(1) == 1 and y.dtype == w_out.dtype
+    for w in (w_out, w_next):
+        assert w is None or (w.dtype == y.dtype and w.numel() == D and w.is_contiguous())
+    if rows is not None:
+        assert rows.dtype == torch.int32 and rows.dim() == 2 and rows.shape[0] == T and rows.is_contiguous()
+    else:
+        assert y.shape[0] == T
+    if y2 is not None:
+        assert y2.shape == (T, D) and y2.stride(1) == 1 and y2.dtype == y.dtype
+        assert y2_gate.dtype == torch.float32 and y2_gate.shape == (T,)
+    h = torch.empty((T, D), dtype=y.dtype, device=x.device) if w_next is not None else None
+    check(_lib_().mi355_layernorm_residual_add(x.data_ptr(), _p(h), y.data_ptr(), max(y.stride(0), D), _p(rows),
+                                               rows.shape[1] if rows is not None else 0, _p(y2), max(y2.stride(0), D) if y2 is not None else 0,
+                                               _p(y2_gate), y2_gate.stride(0) if y2_gate is not None else 0, w_out.data_ptr(), _p(w_next),
+                                               T, D, float(eps), _dt(y), _stream(x)), "layernorm_residual_add")
+    return h
+
+
+def project_f32(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
+    """x [T, K] (row-strided) against a small table [N, K] of the same dtype -> unrounded fp32 [T, N], the same numbers for a row
+    whatever rows lie beside it."""
+    _gpu(x, weight)
+    T, K = x.shape
+    assert x.stride(1) == 1 and weight.dtype == x.dtype and weight.is_contiguous() and weight.shape[1] == K
+    if x.dtype == torch.float32:
+        return moe_router_logits(x.contiguous(), weight)
+    out = torch.empty((T, weight.shape[0]), dtype=torch.float32, device=x.device)
+    check(_lib_().mi355_project_f32(out.data_ptr(), x.data_ptr(), max(x.stride(0), K), weight.data_ptr(), T, weight.shape[0], K, _dt(x),
+                                    _stream(x)), "project_f32")
+    return out
+
+
+def clamped_glu(a: torch.Tensor, limit: float, alpha: float, rows: Optional[torch.Tensor] = None,
+                coef: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """a [P, 2 ff] = [gate | up] -> [P, ff]: g sigmoid(alpha g) (u + 1) with g = min(c gate, limit), u = clamp(c up, -limit, limit).
+    rows int32 / coef fp32 of one shape: only the listed rows are computed, row rows[j] with c = coef[j]; otherwise all, c = 1."""
+    _gpu(a, rows, coef)
+    P, ff2 = a.shape
+    assert a.stride(1) == 1 and ff2 % 2 == 0 and limit >= 0
+    assert (rows is None) == (coef is None)
+    if rows is not None:
+        assert rows.dtype == torch.int32 and coef.dtype == torch.float32 and rows.shape == coef.shape
+        assert rows.is_contiguous() and coef.is_contiguous()
+    out = torch.empty((P, ff2 // 2), dtype=a.dtype, device=a.device)
+    check(_lib_().mi355_clamped_glu(out.data_ptr(), a.data_ptr(), max(a.stride(0), ff2), _p(rows), _p(coef),
+                                    rows.numel() if rows is not None else P, ff2 // 2, float(limit), float(alpha), _dt(a), _stream(a)),
+          "clamped_glu")
+    return out
+
+
+MATRIX_MEMORY_VALUE_BLOCK = 32     # value columns that share one copy of the normaliser (mi355_matrix_memory_value_block)
+
+
+def matrix_memory(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, in_logits: torch.Tensor, forget_logits: torch.Tensor,
+                  in_bias: torch.Tensor, forget_bias: torch.Tensor, out: torch.Tensor, state: torch.Tensor, norm_state: torch.Tensor,
+                  req_to_state: torch.Tensor, req_pool_indices: torch.Tensor, positions: torch.Tensor, q_scale: float, gate_cap: float,
+                  tok_req=None, seg_start=None, seg_len=None) -> torch.Tensor:
+    """Matrix memory with exponential gates over every sequence's tokens of the step: with i = c tanh((in_logits + in_bias) / c),
+    f = logsigmoid(c tanh((forget_logits + forget_bias) / c)), c = gate_cap:  m' = max(f + m, i);  (S, n) <- e^(f + m - m') (S, n) +
+    e^(i - m') (k v^T, k);  out = S^T q / (max(|n . q|, e^-m') + 1e-6), q times q_scale.  q, k [T, H, dk], v [T, H, dv], logits fp32
+    [T, H] (row-strided alike), biases fp32 [H], state fp32 [slots, H, dk, dv], norm_state fp32 [slots, H, blocks, dk + 1]."""
+    _gpu(q, k, v, in_logits, forget_logits, in_bias, forget_bias, out, state, norm_state, req_to_state, req_pool_indices, positions)
+    T, H, dk = q.shape
+    dv = v.shape[2]
+    assert k.shape == q.shape and v.shape[:2] == (T, H) and q.dtype == k.dtype == v.dtype
+    for t in (q, k, v):
+        assert t.stride(2) == 1 and t.stride(1) == t.shape[2], "heads lie side by side in a token's row"
+    for z in (in_logits, forget_logits):
+        assert z.dtype == torch.float32 and z.shape == (T, H) and z.stride(1) == 1 and z.stride(0) == in_logits.stride(0)
+    for z in (in_bias, forget_bias):
+        assert z.dtype == torch.float32 and z.numel() == H and z.is_contiguous()
+    assert out.dtype == torch.float32 and out.shape == (T, H, dv) and out.is_contiguous()
+    assert state.dtype == torch.float32 and state.is_contiguous() and tuple(state.shape[1:]) == (H, dk, dv)
+    blocks = -(-dv // int(_lib_().mi355_matrix_memory_value_block()))
+    assert norm_state.dtype == torch.float32 and norm_state.is_contiguous() and tuple(norm_state.shape) == (state.shape[0], H, blocks, dk + 1)
+    assert req_to_state.dtype == torch.int32 and req_pool_indices.dtype == torch.int64 and positions.dtype == torch.int64
+    _, ss, sl = _seg(tok_req, seg_start, seg_len)
+    B = req_pool_indices.numel()
+    assert seg_start is not None or B == T, "without segments every token is a sequence of its own"
+    check(_lib_().mi355_matrix_memory(out.data_ptr(), state.data_ptr(), norm_state.data_ptr(), q.data_ptr(), k.data_ptr(), v.data_ptr(),
+                                      in_logits.data_ptr(), forget_logits.data_ptr(), in_bias.data_ptr(), forget_bias.data_ptr(),
+                                      req_to_state.data_ptr(), req_pool_indices.data_ptr(), ss, sl, positions.data_ptr(), B, H, dk, dv,
+                                      blocks, q.stride(0), k.stride(0), v.stride(0), max(in_logits.stride(0), H), float(q_scale),
+                                      float(gate_cap), _dt(q), _stream(q)), "matrix_memory")
+    return out

@@ -266,10 +266,17 @@ def gated_residual_add(x, g1, b1, y1, g2=None, b2=None, y2=None):
     x.add_(add)
 
 
-def _rot(v, pos, inv_freq, rot_dims):
+def _rot(v, pos, inv_freq, rot_dims, interleaved=False, rot_mag=1.0):
     half = rot_dims // 2
+    if half == 0:
+        return v.float()
     ang = float(pos) * inv_freq[:half].float()
-    c, s = torch.cos(ang), torch.sin(ang)
+    c, s = torch.cos(ang) * rot_mag, torch.sin(ang) * rot_mag
+    if interleaved:
+        out = v.float().clone()
+        a, b = out[..., 0:rot_dims:2].clone(), out[..., 1:rot_dims:2].clone()
+        out[..., 0:rot_dims:2], out[..., 1:rot_dims:2] = a * c - b * s, b * c + a * s
+        return out
     u, w = v[..., :half].float(), v[..., half:rot_dims].float()
     return torch.cat([u * c - w * s, w * c + u * s, v[..., rot_dims:].float()], -1)
 
@@ -289,6 +296,15 @@ def latent_norms_rope_write(a, q_weight, kv_weight, positions, out_cache_loc, in
     return cq
 
 
+def latent_rows_write(a, q_cols, kv_weight, positions, out_cache_loc, inv_freq, cache, rank, rope_dim, rot_dims, interleaved, rot_mag, eps):
+    for t in range(a.shape[0]):
+        row = a[t].float()
+        c = row[q_cols: q_cols + rank]
+        c = c / torch.sqrt((c * c).mean() + eps) * kv_weight.float()
+        kr = _rot(row[q_cols + rank: q_cols + rank + rope_dim], positions[t], inv_freq, rot_dims, interleaved, rot_mag)
+        cache[int(out_cache_loc[t])] = torch.cat([c, kr]).to(cache.dtype)
+
+
 def latent_window_attention_block_tokens(heads, rank, rope_dim, dtype):
     return 3
 
@@ -298,7 +314,7 @@ def latent_window_attention_splits(tokens, heads, rank, window, max_position, dt
 
 
 def latent_window_attention(qa, qr, cache, out, req_to_token, req_pool_indices, positions, sink, inv_freq, rot_dims, window,
-                            scale, gate=None, tok_req=None, blocks=None, num_splits=1):
+                            scale, gate=None, tok_req=None, blocks=None, num_splits=1, interleaved=False, rot_mag=1.0):
     T, H, rank = qa.shape
     covered = torch.zeros(T, dtype=torch.bool)
     runs = [(t, 1) for t in range(T)] if blocks is None else [(int(a), int(n)) for a, n in blocks.tolist()]
@@ -309,14 +325,16 @@ def latent_window_attention(qa, qr, cache, out, req_to_token, req_pool_indices, 
             b = t if tok_req is None else int(tok_req[t])
             assert blocks is None or int(tok_req[t0]) == b, "a run crosses two sequences"
             p = int(positions[t])
-            lo = max(0, p - window + 1)
+            lo = max(0, p - window + 1) if window > 0 else 0
             slots = req_to_token[int(req_pool_indices[b]), lo: p + 1].long()
             rows = cache[slots].float()                                  # [n_keys, rank + rope]
-            q = torch.cat([qa[t].float(), _rot(qr[t], p, inv_freq, rot_dims)], -1)   # [H, rank + rope]
+            q = torch.cat([qa[t].float(), _rot(qr[t], p, inv_freq, rot_dims, interleaved, rot_mag)], -1)   # [H, rank + rope]
             s = (q @ rows.T) * scale                                     # [H, n_keys]
-            m = torch.maximum(s.max(-1).values, sink.float())
+            m = s.max(-1).values
+            if sink is not None:
+                m = torch.maximum(m, sink.float())
             e = torch.exp(s - m[:, None])
-            pr = e / (e.sum(-1) + torch.exp(sink.float() - m))[:, None]
+            pr = e / (e.sum(-1) + (torch.exp(sink.float() - m) if sink is not None else 0.0))[:, None]
             o = pr @ rows[:, :rank]
             if gate is not None:
                 o = o * torch.sigmoid(gate[t].float())[:, None]
@@ -558,7 +576,7 @@ def head_rmsnorm_gate_act(o, weight, gate, eps, out_dtype, gate_act="silu"):
     T, H, dv = o.shape
     n = o / torch.sqrt((o * o).mean(-1, keepdim=True) + eps)
     if weight is not None:
-        n = n * weight.float()
+        n = n * (weight.float().view(H, dv) if weight.numel() == H * dv else weight.float())
     g = gate.float().reshape(T, H, dv)
     return (n * (torch.sigmoid(g) if gate_act == "sigmoid" else g * torch.sigmoid(g))).reshape(T, H * dv).to(out_dtype)
 
@@ -568,6 +586,8 @@ def _act(z, act):
         return z * torch.sigmoid(z)
     if act == "relu2":
         return torch.clamp(z, min=0.0) ** 2
+    if act == "gelu_erf":
+        return 0.5 * z * (1.0 + torch.erf(z * 0.7071067811865476))
     return z
 
 
@@ -697,3 +717,63 @@ def moe_route_scores(logits, correction, top, n_groups, keep_groups, scale, scor
         sel = s[t, order]
         w[t] = (sel / (sel.sum() + 1e-20) if renorm else sel) * scale
     return ids, w
+
+
+# ------------------------------------------------------- layer norms around every sublayer, matrix memory, clamped experts.
+# Token-by-token restatements of what the header says of each kernel; they share nothing with oracle/silatar_ref.py.
+def layernorm_residual_add(x, y, w_out, w_next, eps, rows=None, y2=None, y2_gate=None):
+    T = x.shape[0]
+    h = torch.empty_like(x)
+    for t in range(T):
+        b = y[t].float() if rows is None else sum(y[int(r)].float() for r in rows[t])
+        if y2 is not None:
+            b = b + torch.sigmoid(y2_gate[t]) * y2[t].float()
+        x[t] += _ln(b, w_out, eps)
+        if w_next is not None:
+            h[t] = _ln(x[t], w_next, eps)
+    return None if w_next is None else h.to(w_next.dtype)
+
+
+def project_f32(x, weight):
+    return F.linear(x.float(), weight.float())
+
+
+def clamped_glu(a, limit, alpha, rows=None, coef=None):
+    P, ff = a.shape[0], a.shape[1] // 2
+    out = torch.full((P, ff), float("nan"), dtype=a.dtype)        # a row that nobody lists must not be read
+    todo = [(p, 1.0) for p in range(P)] if rows is None else [(int(p), float(c)) for p, c in zip(rows.reshape(-1), coef.reshape(-1))]
+    for p, c in todo:
+        g = torch.clamp(c * a[p, :ff].float(), max=limit)
+        u = torch.clamp(c * a[p, ff:].float(), -limit, limit)
+        out[p] = (g * torch.sigmoid(alpha * g) * (u + 1.0)).to(a.dtype)
+    return out
+
+
+MATRIX_MEMORY_VALUE_BLOCK = 32
+
+
+def matrix_memory(q, k, v, in_logits, forget_logits, in_bias, forget_bias, out, state, norm_state, req_to_state, req_pool_indices,
+                  positions, q_scale, gate_cap, tok_req=None, seg_start=None, seg_len=None):
+    T, H, dk = q.shape
+    S = n = m = None
+    for t, (b, first, last) in enumerate(_segments(T, tok_req, seg_start, seg_len)):
+        slot = int(req_to_state[int(req_pool_indices[b])])
+        if first:
+            fresh = int(positions[t]) == 0
+            S = torch.zeros_like(state[slot]) if fresh else state[slot].clone()
+            nm = torch.zeros_like(norm_state[slot, :, 0]) if fresh else norm_state[slot, :, 0].clone()
+            n, m = nm[:, :dk], nm[:, dk]
+        i = gate_cap * torch.tanh((in_logits[t] + in_bias) / gate_cap)
+        f = F.logsigmoid(gate_cap * torch.tanh((forget_logits[t] + forget_bias) / gate_cap))
+        m1 = torch.maximum(f + m, i)
+        keep, write = torch.exp(f + m - m1)[:, None], torch.exp(i - m1)[:, None]
+        kk, qq = k[t].float(), q[t].float() * q_scale
+        S = keep[:, :, None] * S + (write * kk)[:, :, None] * v[t].float()[:, None, :]
+        n = keep * n + write * kk
+        m = m1
+        den = torch.maximum((n * qq).sum(-1).abs(), torch.exp(-m)) + 1e-6
+        out[t] = (S * qq[:, :, None]).sum(1) / den[:, None]
+        if last:
+            state[slot] = S
+            norm_state[slot] = torch.cat([n, m[:, None]], 1)[:, None, :].expand_as(norm_state[slot])
+    return out
