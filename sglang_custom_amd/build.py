@@ -48,6 +48,8 @@ FAMILY_SOURCES = {
                 "moe_ops.hip", "conv_ops.hip", "attn_window.hip"],
     "Fudonex": ["elementwise.hip", "index_ops.hip", "gemm.hip", "gemm_tiled.hip", "postnorm_ops.hip", "recurrence.hip",
                 "conv_ops.hip", "attn_window.hip"],
+    "Silatar": ["elementwise.hip", "index_ops.hip", "gemm.hip", "gemm_tiled.hip", "stream_ops.hip", "attn_latent.hip", "postnorm_ops.hip",
+                "recurrence.hip", "moe_ops.hip", "conv_ops.hip", "mla_proj.hip"],
 }
 PARTIAL_MARK = LIB + ".partial"
 

@@ -32,6 +32,9 @@ class ModelConfig:
         if self.architecture == "Fudonex":
             self._init_fudonex(c, dtype, context_length, quantization)
             return
+        if self.architecture == "Silatar":
+            self._init_silatar(c, dtype, context_length, quantization)
+            return
         self.hidden_size = c["hidden_size"]
         self.num_hidden_layers = c["num_hidden_layers"]
         self.num_attention_heads = c["num_attention_heads"]
@@ -290,6 +293,65 @@ class ModelConfig:
         self.recurrent_layer_shapes = [None if s["type"] == "attention" else
                                        (s["mixer"]["heads"], s["mixer"]["state"] if s["type"] == "mamba2" else s["mixer"]["dim"],
                                         s["mixer"]["vdim"]) for s in layers]
+
+    def _init_silatar(self, c: dict, dtype: str, context_length: Optional[int], quantization: Optional[str]) -> None:
+        """The Silatar design: "layers" lists the layers one by one, {"type": "latent_attention" | "mlstm", "mixer": {...}, "mlp":
+        {"kind": "dense", "ff"} | {"kind": "moe", "expert": {"ff", "limit"}, "router": {"experts", "top"}, "shared": {"ff", "limit"}}
+        | null}; widths under "width" / "vocab", the norms' epsilon under "norm", the cap of the logits under "logit_softcap".
+        "loop" {"start", "stop", "times"}: layers start .. stop - 1 run `times` times in a row with the same weights.  layer_runs
+        lists the layer of every run; caches and states belong to runs, not to layers: latent_kv (rank, rope width) of the
+        attention runs, recurrent_layer_shapes (heads, key width, value width) of the others, None elsewhere.  Layers may differ
+        in every size."""
+        layers = c["layers"]
+        for i, spec in enumerate(layers):
+            m, mlp = spec["mixer"], spec.get("mlp")
+            if spec["type"] == "latent_attention":
+                rot = m.get("rot")
+                if rot and (rot["dims"] % 2 or not 0 <= rot["dims"] <= m["rot_dim"]):
+                    raise ValueError(f"Silatar layer {i}: rotation over {rot['dims']} of {m['rot_dim']} features")
+            elif spec["type"] == "mlstm":
+                if not m["gate_cap"] > 0:
+                    raise ValueError(f"Silatar layer {i}: gate_cap {m['gate_cap']} is not positive")
+            else:
+                raise ValueError(f"Silatar layer {i}: unknown mixer type {spec['type']!r}")
+            if mlp is not None:
+                if mlp.get("kind") not in ("dense", "moe"):
+                    raise ValueError(f"Silatar layer {i}: unknown feed-forward kind {mlp.get('kind')!r}")
+                if mlp["kind"] == "moe" and not 1 <= mlp["router"]["top"] <= mlp["router"]["experts"]:
+                    raise ValueError(f"Silatar layer {i}: {mlp['router']['top']} of {mlp['router']['experts']} experts")
+        n = len(layers)
+        loop = c.get("loop") or {"start": 0, "stop": 0, "times": 1}
+        a, b, times = int(loop["start"]), int(loop["stop"]), int(loop["times"])
+        if not (0 <= a <= b <= n and times >= 1):
+            raise ValueError(f"Silatar: a loop over layers {a} .. {b - 1}, {times} times, of {n} layers")
+        self.layer_runs = list(range(a)) + list(range(a, b)) * times + list(range(b, n))
+        self.layer_specs = layers
+        self.hidden_size = c["width"]
+        self.vocab_size = c["vocab"]
+        self.num_hidden_layers = len(self.layer_runs)       # what pools count: caches and states belong to runs
+        att = [s["mixer"] for s in layers if s["type"] == "latent_attention"]
+        self.num_attention_heads = max([m["heads"] for m in att] or [1])
+        self.num_key_value_heads = 1
+        self.head_dim = max([m["kv_rank"] + m["rot_dim"] for m in att] or [1])
+        self.v_head_dim = max([m["kv_rank"] for m in att] or [1])
+        self.intermediate_size = max([s["mlp"]["ff"] if s["mlp"]["kind"] == "dense" else s["mlp"]["expert"]["ff"]
+                                      for s in layers if s.get("mlp")] or [0])
+        self.rms_norm_eps = c["norm"]["eps"]
+        cap = c.get("logit_softcap")
+        self.final_logit_softcapping = float(cap) if cap else None
+        self.rope_theta = None
+        self.rope_scaling = None
+        self.tie_word_embeddings = False
+        self.max_position_embeddings = context_length or 131072     # the design fixes no longest sequence
+        self.context_len = self.max_position_embeddings
+        self.quantization = quantization
+        self.dtype = _DTYPES.get(dtype) or torch.bfloat16
+        self.is_encoder_decoder = False
+        runs = [layers[i] for i in self.layer_runs]
+        self.needs_sequence_state = any(s["type"] == "mlstm" for s in runs)
+        self.latent_kv = [(s["mixer"]["kv_rank"], s["mixer"]["rot_dim"]) if s["type"] == "latent_attention" else None for s in runs]
+        self.recurrent_layer_shapes = [(s["mixer"]["heads"], s["mixer"]["dim"], s["mixer"]["vdim"]) if s["type"] == "mlstm" else None
+                                       for s in runs]
 
     @classmethod
     def from_path(cls, model_path: str, **kw) -> "ModelConfig":

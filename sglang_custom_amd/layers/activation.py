@@ -1,5 +1,8 @@
 """SiluAndMul (python/sglang/srt/layers/activation.py:55-65): x [.., 2d] -> [.., d]; Activation: a plain elementwise
-function of a projection's output ("silu", or "relu2", the square of relu)."""
+function of a projection's output ("silu", "relu2" -- the square of relu -- or "gelu_erf"); ClampedGLU: a gated unit whose
+two halves are clamped."""
+from typing import Optional
+
 import torch
 
 from ..custom_op import CustomOp
@@ -24,9 +27,21 @@ class GeluTanhAndMul(CustomOp):
 class Activation(CustomOp):
     def __init__(self, kind: str):
         super().__init__()
-        assert kind in ("silu", "relu2")
+        assert kind in ("silu", "relu2", "gelu_erf")
         self.kind = kind
 
     def forward_hip(self, x: torch.Tensor) -> torch.Tensor:
         """x [T, d] (row-strided: a column block of a wider projection will do) -> contiguous [T, d]."""
         return get_ops().activation(x, self.kind)
+
+
+class ClampedGLU(CustomOp):
+    """[gate | up] -> g sigmoid(alpha g) (u + 1) with g = min(c gate, limit), u = clamp(c up, -limit, limit).  c = 1, or per listed
+    row (rows, coef): a factor on the input of the bias-free projections in front, which they commute with."""
+
+    def __init__(self, limit: float, alpha: float = 1.702):
+        super().__init__()
+        self.limit, self.alpha = float(limit), float(alpha)
+
+    def forward_hip(self, x: torch.Tensor, rows: Optional[torch.Tensor] = None, coef: Optional[torch.Tensor] = None) -> torch.Tensor:
+        return get_ops().clamped_glu(x, self.limit, self.alpha, rows=rows, coef=coef)

@@ -72,7 +72,7 @@ class Mi355AttnBackend(AttentionBackend):
             self.num_kv_head = (self.num_head + 15) // 16
         # value width as the pool stores it (an MLA pool's value is the first kv_lora_rank features of
         # its rows); read from the buffer so that any pool with the reference's accessors works
-        self.v_head_dim = (cfg.v_head_dim if self.is_layered
+        self.v_head_dim = (cfg.v_head_dim if self.is_layered or self.is_latent_window
                            else model_runner.token_to_kv_pool.get_value_buffer(0).shape[-1])
         self.max_context_len = int(getattr(cfg, "context_len", 0) or self.req_to_token.shape[1])
         sw = getattr(model_runner, "sliding_window_size", None)
@@ -295,15 +295,16 @@ class Mi355AttnBackend(AttentionBackend):
             cache[bq] = host.contiguous().to(self.device, non_blocking=True)
         return cache[bq]
 
-    def forward_latent_window(self, qa, qr, gate, layer, forward_batch, out):
-        """qa [T, H, rank] absorbed queries, qr [T, H, rope] unrotated, gate [T, H] logits or None -> out [T, H, rank].
+    def forward_latent_window(self, qa, qr, gate, layer, forward_batch, out, cache_layer=None):
+        """qa [T, H, rank] absorbed queries, qr [T, H, rope] unrotated, gate [T, H] logits or None -> out [T, H, rank], over
+        the rows of cache_layer (the layer's own by default), its last layer.window tokens or (0) every earlier one.
         The new tokens' rows are in the cache already (ops.latent_norms_rope_write); prefill portions, decode steps and
         mixed batches are the same launch, told apart only by the list of token runs."""
         ops = get_ops()
         bq = ops.latent_window_attention_block_tokens(layer.tp_q_head_num, layer.kv_rank, layer.rope_dim, qa.dtype)
         if bq <= 0:
             raise NotImplementedError(f"latent window attention: rank {layer.kv_rank} + rope {layer.rope_dim} is not served")
-        cache = forward_batch.token_to_kv_pool.get_key_buffer(layer.layer_id)
+        cache = forward_batch.token_to_kv_pool.get_key_buffer(layer.layer_id if cache_layer is None else cache_layer)
         splits = 1
         if forward_batch.forward_mode.is_decode() and forward_batch.seq_lens_cpu is not None:
             # a decode step has few workgroups: long windows are cut into key ranges that a second launch merges
@@ -311,8 +312,9 @@ class Mi355AttnBackend(AttentionBackend):
                                                         int(forward_batch.seq_lens_cpu.max()) - 1, qa.dtype)
         return ops.latent_window_attention(
             qa, qr, cache, out, forward_batch.req_to_token_pool.req_to_token, forward_batch.req_pool_indices,
-            forward_batch.positions, layer.sink.data, layer.inv_freq, layer.rot_dims, layer.window, layer.scaling, gate=gate,
-            tok_req=forward_batch.token_req_index(), blocks=self._latent_blocks(forward_batch, bq), num_splits=splits)
+            forward_batch.positions, layer.sink.data if layer.sink is not None else None, layer.inv_freq, layer.rot_dims, layer.window,
+            layer.scaling, gate=gate, tok_req=forward_batch.token_req_index(), blocks=self._latent_blocks(forward_batch, bq),
+            num_splits=splits, interleaved=layer.interleaved, rot_mag=layer.rot_mag)
 
     # ---- causal attention with sigmoid weights (no softmax) over per-layer key / value buffers ----
     def forward_sigmoid(self, q, layer, forward_batch, out):

@@ -14,7 +14,8 @@ from ..distributed.parallel_state import (
     get_tensor_model_parallel_world_size,
     tensor_model_parallel_all_reduce,
 )
-from .quantization.unquant import PendingAllReduce, UnquantizedLinearMethod
+from ..ops_backend import get_ops
+from .quantization.unquant import SKINNY_MAX_M, PendingAllReduce, UnquantizedLinearMethod
 
 
 class LinearBase(nn.Module):
@@ -36,6 +37,30 @@ class ReplicatedLinear(LinearBase):
 
     def forward(self, x):
         return self.quant_method.apply(self, x), None
+
+
+class PerHeadLinear(nn.Module):
+    """One small matrix per head: y[t, h] = W[h] x[t, h] (the expansions of a latent in absorbed attention).  Kept twice: weight
+    [H, n, k] with the reduction contiguous, which the one-launch kernel of decode-sized steps reads (ops.mla_absorb), and
+    weight_kn [H, k, n], the right operand of the batched product that serves everything else."""
+
+    def __init__(self, heads: int, input_size: int, output_size: int, dtype, device):
+        super().__init__()
+        self.heads, self.input_size, self.output_size = heads, input_size, output_size
+        self.weight = nn.Parameter(torch.zeros(heads, output_size, input_size, dtype=dtype, device=device), requires_grad=False)
+        self.weight_kn = None
+
+    def process_weights_after_loading(self) -> None:
+        self.weight_kn = self.weight.data.transpose(1, 2).contiguous()
+
+    def forward(self, x: torch.Tensor) -> torch.Tensor:
+        """x [T, H, k] (token and head strides free, features contiguous) -> [T, H, n], possibly a permuted view."""
+        ops = get_ops()
+        T = x.shape[0]
+        if (T <= SKINNY_MAX_M and x.stride(2) == 1 and x.stride(0) % 8 == 0 and x.stride(1) % 8 == 0 and x.stride(0) >= x.stride(1)
+                and x.data_ptr() % 16 == 0 and ops.mla_absorb_supported(T, self.output_size, self.input_size, 0, x.dtype)):
+            return ops.mla_absorb(x, self.weight.data)
+        return torch.bmm(x.transpose(0, 1), self.weight_kn).transpose(0, 1)
 
 
 class QKVParallelLinear(LinearBase):

@@ -24,10 +24,19 @@ size, dt_t = softplus(z_t + dt_bias), a_t = exp(-exp(rate_log_h) dt_t):
 
 B and C (the keys and the queries) may be shared by groups of heads.
 
+MatrixMemory: the same hand-off for a matrix memory with exponential gates, i = c tanh((zi + bi) / c) and
+f = logsigmoid(c tanh((zf + bf) / c)) from fp32 logits of one number per head:
+
+    m_t = max(f + m_{t-1}, i);   (S, n)_t = e^(f + m_{t-1} - m_t) (S, n)_{t-1} + e^(i - m_t) (k v^T, k)
+    o_t = S_t^T q / (max(|n_t . q|, e^(-m_t)) + 1e-6)
+
+whose normaliser n and running maximum m live beside the matrices (SequenceStatePool.vectors[layer]).  Its state belongs to a
+cache layer given with every call, so that one set of weights can run several times per step over states of their own.
+
 GatedGroupNorm: y * silu(gate), THEN an RMS norm over `groups` equal parts of the row, times a weight.
 
-HeadNormGate: the recurrence's fp32 output per head divided by its root mean square (times a weight shared by the heads,
-if there is one), times silu(gate) or sigmoid(gate), in the activation dtype for the output projection."""
+HeadNormGate: the recurrence's fp32 output per head divided by its root mean square (times a weight shared by the heads or,
+with `heads`, one per head, if there is one), times silu(gate) or sigmoid(gate), in the activation dtype for the output projection."""
 from typing import Optional
 
 import torch
@@ -113,20 +122,47 @@ class GatedDeltaRule(nn.Module):
         return out
 
 
+class MatrixMemory(nn.Module):
+    def __init__(self, num_heads: int, key_dim: int, value_dim: int, gate_cap: float, device, q_scale: float = 1.0):
+        super().__init__()
+        assert gate_cap > 0
+        self.num_heads, self.key_dim, self.value_dim = num_heads, key_dim, value_dim
+        self.gate_cap, self.q_scale = float(gate_cap), float(q_scale)
+        # fp32 whatever the model dtype: they enter the gates
+        self.in_bias = nn.Parameter(torch.zeros(num_heads, dtype=torch.float32, device=device), requires_grad=False)
+        self.forget_bias = nn.Parameter(torch.zeros(num_heads, dtype=torch.float32, device=device), requires_grad=False)
+
+    def state_vectors(self):
+        """Shape of the per-sequence state beside the matrices: (n, m) once per block of value columns."""
+        return (self.num_heads, -(-self.value_dim // get_ops().MATRIX_MEMORY_VALUE_BLOCK), self.key_dim + 1)
+
+    def forward(self, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate_logits: torch.Tensor, forward_batch,
+                cache_layer: int) -> torch.Tensor:
+        """q, k [T, H, dk], v [T, H, dv] (any token stride), gate_logits fp32 [T, 2 H] = [input | forget] -> fp32 [T, H, dv]."""
+        st = forward_batch.seq_state
+        H = self.num_heads
+        out = torch.empty((q.shape[0], H, self.value_dim), dtype=torch.float32, device=q.device)
+        get_ops().matrix_memory(q, k, v, gate_logits[:, :H], gate_logits[:, H:], self.in_bias.data, self.forget_bias.data, out,
+                                st.pool.matrices[cache_layer], st.pool.vectors[cache_layer], st.req_to_state, st.req_pool_indices,
+                                forward_batch.positions, self.q_scale, self.gate_cap, **st.segments())
+        return out
+
+
 class HeadNormGate(nn.Module):
-    def __init__(self, value_dim: int, eps: float, dtype, device, with_weight: bool, gate_act: str = "silu"):
+    def __init__(self, value_dim: int, eps: float, dtype, device, with_weight: bool, gate_act: str = "silu", heads: int = 1):
         super().__init__()
         assert gate_act in ("silu", "sigmoid")
         self.gate_act = gate_act
         self.eps = float(eps)
         self.out_dtype = dtype
-        self.weight = (nn.Parameter(torch.ones(value_dim, dtype=dtype, device=device), requires_grad=False)
+        self.per_head = heads > 1
+        self.weight = (nn.Parameter(torch.ones(heads * value_dim, dtype=dtype, device=device), requires_grad=False)
                        if with_weight else None)
 
     def forward(self, o: torch.Tensor, gate: torch.Tensor) -> torch.Tensor:
         """o fp32 [T, H, dv], gate [T, H * dv] logits (row-strided) -> [T, H * dv]."""
         w = self.weight.data if self.weight is not None else None
-        if self.gate_act == "silu":
+        if self.gate_act == "silu" and not self.per_head:
             return get_ops().head_rmsnorm_gate(o, w, gate, self.eps, self.out_dtype)
         return get_ops().head_rmsnorm_gate_act(o, w, gate, self.eps, self.out_dtype, self.gate_act)
 

@@ -7,6 +7,10 @@ reference, whose models norm before their sublayers and keep the residual in the
                       writes the activation-dtype copy of the new x that the next projections read.
   NormedResidualAdd   x <- x + mult * ls * y / sqrt(mean(y^2) + eps) * (offset + w) in place, same second output: a norm on a
                       sublayer's OUTPUT; offset 1 for a weight stored around zero, ls an optional per-channel layer scale.
+  LayerNormResidualAdd  x <- x + LN(y) w in place, LN the layer norm without bias, and in the same launch the layer norm in front
+                      of whatever reads the stream next: h = LN(x) w_next.  y may be the sum of a token's expert rows plus a
+                      gated second branch.  Which norm comes next is the caller's: layers may run in another order than they
+                      are stored in.
 
 groups, eps and c are constructor arguments; all arithmetic is fp32 whatever the activation dtype."""
 from typing import Optional
@@ -48,3 +52,15 @@ class NormedResidualAdd(nn.Module):
             return get_ops().rmsnorm_residual_add(x, y, self.weight.data, self.eps)
         return get_ops().rmsnorm_residual_add(x, y, self.weight.data, self.eps, offset=self.offset, mult=self.mult,
                                               layer_scale=self.layer_scale.data if self.layer_scale is not None else None)
+
+
+class LayerNormResidualAdd(nn.Module):
+    def __init__(self, hidden: int, eps: float, dtype, device):
+        super().__init__()
+        self.eps = float(eps)
+        self.weight = nn.Parameter(torch.ones(hidden, dtype=dtype, device=device), requires_grad=False)
+
+    def forward(self, x: torch.Tensor, y: torch.Tensor, next_weight: Optional[torch.Tensor], rows: Optional[torch.Tensor] = None,
+                y2: Optional[torch.Tensor] = None, y2_gate: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+        """x fp32 [T, D], updated in place; returns LN(x) * next_weight in the weight's dtype."""
+        return get_ops().layernorm_residual_add(x, y, self.weight.data, next_weight, self.eps, rows=rows, y2=y2, y2_gate=y2_gate)

@@ -204,7 +204,8 @@ class SequenceStatePool:
     """State that a sequence carries from one step to the next, for models that have such (no counterpart in the
     reference, whose models keep nothing but KV): per slot the last token id, per layer one fp32 row of the
     model's width (the previous token's normed input of a token-shift layer) and, for layers with a linear
-    recurrence, one fp32 matrix per head ([heads, key width, value width], `matrices[layer]`; layers may differ), and
+    recurrence, one fp32 matrix per head ([heads, key width, value width], `matrices[layer]`; layers may differ), for
+    recurrences with a normaliser further fp32 numbers beside the matrices (`vectors[layer]`, any shape per slot), and
     for every short causal convolution the last taps - 1 inputs of its channels (`convs[key]`, fp32
     [slots, taps - 1, channels], row taps - 2 the most recent; the keys are the model's own).
     A request holds one slot from its first prefill portion until it finishes or is retracted; what a freed slot
@@ -212,7 +213,7 @@ class SequenceStatePool:
     handed out."""
 
     def __init__(self, size: int, layer_num: int, hidden: int, device: str, matrices: Optional[dict] = None,
-                 convs: Optional[dict] = None):
+                 convs: Optional[dict] = None, vectors: Optional[dict] = None):
         self.size = size
         self.layer_num = layer_num
         self.hidden = hidden
@@ -221,13 +222,15 @@ class SequenceStatePool:
         self.prev_token = torch.zeros(size + 1, dtype=torch.int32, device=device)
         self.matrices = {layer: torch.zeros((size + 1, h, dk, dv), dtype=torch.float32, device=device)
                          for layer, (h, dk, dv) in (matrices or {}).items()}
+        self.vectors = {layer: torch.zeros((size + 1,) + tuple(shape), dtype=torch.float32, device=device)
+                        for layer, shape in (vectors or {}).items()}
         self.convs = {key: torch.zeros((size + 1, max(taps - 1, 0), channels), dtype=torch.float32, device=device)
                       for key, (taps, channels) in (convs or {}).items()}
         self.free_slots = list(range(1, size + 1))
 
     def get_state_size_bytes(self) -> int:
         return (self.rows.numel() * 4 + sum(m.numel() * 4 for m in self.matrices.values())
-                + sum(c.numel() * 4 for c in self.convs.values()))
+                + sum(c.numel() * 4 for c in self.convs.values()) + sum(v.numel() * 4 for v in self.vectors.values()))
 
     def available_size(self) -> int:
         return len(self.free_slots)
@@ -246,10 +249,11 @@ class SequenceStatePool:
 
 class LatentTokenToKVPool:
     """Latent KV cache whose layers may differ in width: per layer one row [c (rank_l) | rotated rope key (rope_l)]
-    per token, [size + page_size, rank_l + rope_l]; slot 0 is the sink row of padded tokens, as in the other pools.
+    per token, [size + page_size, rank_l + rope_l], or none at all (widths[l] is None: a layer that keeps no rows, e.g. one
+    with a recurrent mixer); slot 0 is the sink row of padded tokens, as in the other pools.
     (MLATokenToKVPool is the special case of equal layers, kept for the DeepSeek kernels that assume one width.)"""
 
-    def __init__(self, size: int, page_size: int, dtype: torch.dtype, widths: List[Tuple[int, int]], device: str):
+    def __init__(self, size: int, page_size: int, dtype: torch.dtype, widths: List[Optional[Tuple[int, int]]], device: str):
         self.size = size
         self.page_size = page_size
         self.dtype = dtype
@@ -258,10 +262,10 @@ class LatentTokenToKVPool:
         self.layer_num = len(widths)
         self.head_num = 1
         self.device = device
-        self.kv_buffer = [torch.zeros((size + page_size, r + d), dtype=dtype, device=device) for r, d in widths]
+        self.kv_buffer = [None if w is None else torch.zeros((size + page_size, w[0] + w[1]), dtype=dtype, device=device) for w in widths]
 
     def get_kv_size_bytes(self) -> int:
-        return sum(b.numel() * b.element_size() for b in self.kv_buffer)
+        return sum(b.numel() * b.element_size() for b in self.kv_buffer if b is not None)
 
     def get_key_buffer(self, layer_id: int) -> torch.Tensor:
         return self.kv_buffer[layer_id]

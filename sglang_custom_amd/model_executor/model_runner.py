@@ -120,7 +120,7 @@ class ModelRunner:
             raise ValueError(f"kv_cache_dtype {kvd!r}: expected 'auto' or 'fp8_e4m3'")
         self.kv_cache_dtype = torch.float8_e4m3fn if kvd == "fp8_e4m3" else self.dtype
         mla = getattr(cfg, "is_mla", False)
-        latent = getattr(cfg, "latent_kv", None)     # per-layer (rank, rope width) of a latent cache with unequal layers
+        latent = getattr(cfg, "latent_kv", None)     # per-layer (rank, rope width), or None, of a latent cache with unequal layers
         layered = getattr(cfg, "kv_layer_shapes", None)   # per-layer (kv heads, key width, value width) or None per layer
         if layered is not None:
             cell = max(1, sum(h * (dk + dv) for h, dk, dv in filter(None, layered))) * torch.finfo(self.kv_cache_dtype).bits // 8
@@ -130,7 +130,7 @@ class ModelRunner:
                 for p in (sizes or ()) if s is not None else ():
                     cell += -(-s[0] * (s[1] + s[2]) * (torch.finfo(self.kv_cache_dtype).bits // 8) // (p if page_ % p == 0 else 1))
         elif latent is not None:
-            cell = sum(r + d for r, d in latent) * torch.finfo(self.kv_cache_dtype).bits // 8
+            cell = max(1, sum(r + d for r, d in filter(None, latent))) * torch.finfo(self.kv_cache_dtype).bits // 8
         elif mla:
             # one latent row per token and layer (model_runner.py:950-957)
             cell = (cfg.kv_lora_rank + cfg.qk_rope_head_dim) * cfg.num_hidden_layers * torch.finfo(self.kv_cache_dtype).bits // 8
