@@ -82,8 +82,12 @@ def make_weights(cfg, seed=0):
             w[x + "uk"] = rnd(H * d, m["kv_rank"], std=1.5 * m["kv_rank"] ** -0.5)
             w[x + "uv"] = rnd(H * dv, m["kv_rank"], std=m["kv_rank"] ** -0.5)
         else:
-            for n, rows in (("q", H * d), ("k", H * d), ("v", H * dv), ("g", H * dv)):
+            for n, rows in (("q", H * d), ("v", H * dv), ("g", H * dv)):
                 w[x + n] = rnd(rows, D, std=D ** -0.5)
+            # keys that resemble the queries: a token's own write then always shows in its read-out.  With independent ones the
+            # terms of a read-out now and then nearly cancel, and the norm that follows divides the rounding of 16-bit inputs by
+            # the small rest (any 16-bit implementation shows those rows)
+            w[x + "k"] = (w[x + "q"].float() + 0.5 * rnd(H * d, D, std=D ** -0.5).float()).to(torch.bfloat16)
             for n, mean in (("i", -0.5), ("f", 2.0)):
                 w[x + n] = rnd(H, D, std=2 * D ** -0.5)
                 w[x + n + ".b"] = rnd(H, std=0.7, mean=mean)
