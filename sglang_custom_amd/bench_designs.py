@@ -854,3 +854,226 @@ def run_fudonex(size: str, dtype: str = "bfloat16", steps: int = 32, prefill_bs:
     out["stream_decode"] = fudonex_stream_kernels(s, decode_bs, decode_bs)
     out["stream_prefill"] = fudonex_stream_kernels(s, prefill_bs * prefill_len, prefill_bs)
     return out
+
+
+# ------------------------------------------------------------------------------------------------ Silatar beside Verozen and Seturax
+# Silatar shares half of its layers with each of two models of the package, so it is compared twice, at equal width, depth,
+# vocabulary, heads and head widths: its matrix-memory / mixture layers beside Verozen (a linear recurrence with one matrix per
+# head and sequence, a top-k mixture on an fp32 stream; an expert of three matrices of ff beside one of two of 1.5 ff, and
+# Silatar's shared expert counted as one more chosen expert of Verozen's), and its latent attention with dense feed-forwards
+# beside Seturax (the same cache rows; a window as long as the context; two matrices of 1.5 ff beside three of ff).
+SILATAR_SIZES = {
+    "si2048": dict(width=2048, heads=16, nope=128, rope=64, v=128, kv_rank=512, q_rank=1536, rec_heads=16, rec_dim=64, rec_vdim=128, experts=32,
+                   top=3, eff=1024, ff=5632, layers=4, vocab=32768),
+    "si4096": dict(width=4096, heads=32, nope=128, rope=64, v=128, kv_rank=512, q_rank=1536, rec_heads=32, rec_dim=64, rec_vdim=128, experts=64,
+                   top=7, eff=1024, ff=11264, layers=4, vocab=32768),
+    "sitiny": dict(width=320, heads=8, nope=32, rope=16, v=32, kv_rank=64, q_rank=96, rec_heads=4, rec_dim=32, rec_vdim=64, experts=12, top=2,
+                   eff=64, ff=512, layers=4, vocab=2048),
+}
+
+
+def silatar_config(s: dict, kind: str) -> dict:
+    """kind "mixture": matrix memory and latent attention with mixtures; "latent": latent attention with dense feed-forwards."""
+    att = dict(type="latent_attention",
+               mixer=dict(heads=s["heads"], dim=s["nope"], rot_dim=s["rope"], vdim=s["v"], kv_rank=s["kv_rank"], scale=(s["nope"] + s["rope"]) ** -0.5,
+                          rot=dict(base=10000.0, dims=s["rope"], scaling=dict(factor=8.0, original=4096, fast=24.0, slow=2.0))))
+    mem = dict(type="mlstm", mixer=dict(heads=s["rec_heads"], dim=s["rec_dim"], vdim=s["rec_vdim"], gate_cap=15.0))
+    if kind == "mixture":
+        mlp = dict(kind="moe", router=dict(experts=s["experts"], top=s["top"]), expert=dict(ff=s["eff"], limit=7.0), shared=dict(ff=s["eff"], limit=7.0))
+        order = [mem, att, mem, mem]
+    else:
+        mlp = dict(kind="dense", ff=s["ff"] * 3 // 2)
+        order = [att]
+    return dict(architecture="Silatar", vocab=s["vocab"], width=s["width"], norm=dict(eps=1e-6), logit_softcap=30.0,
+                layers=[dict(order[i % len(order)], mlp=mlp) for i in range(s["layers"])])
+
+
+def _silatar_peers(s: dict, window: int):
+    vz = verozen_config(dict(s, kv_heads=max(1, s["heads"] // 4), dim=s["v"], top=s["top"] + 1, groups=1, keep=1, ff=s["eff"] * 3 // 2, side=0, norm_groups=1,
+                             gate_rank=64))
+    vz.pop("token_side")
+    return vz, seturax_config(dict(s, window=window))
+
+
+def silatar_mixer_kernels(s: dict, bs: int, ctx: int, prefill_bs: int, prefill_len: int) -> dict:
+    """Token mixers alone, bf16, each beside the like launch of the closest model on the same shapes.  Latent attention without and
+    with a window that covers everything, sink and gate (decode: bytes = every visible row once per sequence; prefill: flops
+    2 (2 rank + rope) per visible pair and head); the cache row's launch; the per-head expansions as one launch and as a
+    batched library product; the matrix memory beside the recurrence with one decay per head (decode: the matrices' bytes, read
+    and written; prefill: fp32 vector flops, 6 per matrix element and token)."""
+    from . import ops
+    from .layers.rotary_embedding import scaled_pair_inv_freq
+
+    dev, dt = "cuda", torch.bfloat16
+    H, rank, rope, nope = s["heads"], s["kv_rank"], s["rope"], s["nope"]
+    R = rank + rope
+    g = torch.Generator(device=dev).manual_seed(0)
+    f, mag = scaled_pair_inv_freq(10000.0, rope, dict(factor=8.0, original=4096, fast=24.0, slow=2.0))
+    f = f.to(dev)
+    sink = torch.zeros(H, device=dev)
+    T = prefill_bs * prefill_len
+    ss = torch.arange(0, T, prefill_len, device=dev, dtype=torch.int32)
+    sl = torch.full((prefill_bs,), prefill_len, device=dev, dtype=torch.int32)
+    tok_req = torch.repeat_interleave(torch.arange(prefill_bs, device=dev, dtype=torch.int32), prefill_len)
+    res = {}
+    for phase, n, nb, per, reps in (("decode", bs, bs, ctx, 20), ("prefill", T, prefill_bs, prefill_len, 5)):
+        cache = torch.randn(nb * per + 8, R, device=dev, generator=g).to(dt)
+        rtt = (torch.arange(nb * per, device=dev, dtype=torch.int32) + 1).view(nb, per)
+        rpi = torch.arange(nb, device=dev)
+        qa = torch.randn(n, H, rank, device=dev, generator=g).to(dt)
+        qr = torch.randn(n, H, rope, device=dev, generator=g).to(dt)
+        gate = torch.randn(n, H, device=dev, generator=g).to(dt)
+        out = torch.empty_like(qa)
+        if phase == "decode":
+            pos = torch.full((n,), per - 1, device=dev, dtype=torch.int64)
+            kw = dict(num_splits=ops.latent_window_attention_splits(n, H, rank, 0, per - 1, dt))
+            pairs = nb * per
+        else:
+            pos = torch.arange(per, device=dev).repeat(nb)
+            bq = ops.latent_window_attention_block_tokens(H, rank, rope, dt)
+            starts = torch.cat([torch.stack([torch.arange(0, per, bq), torch.clamp(per - torch.arange(0, per, bq), max=bq)], 1) + torch.tensor([[i * per, 0]])
+                                for i in range(nb)])
+            kw = dict(tok_req=tok_req, blocks=starts.to(torch.int32).to(dev))
+            pairs = nb * per * (per + 1) // 2
+        for name, args, extra in (("silatar", (None, f, rope, 0), dict(interleaved=True, rot_mag=mag)), ("seturax", (sink, f, rope, per), dict(gate=gate))):
+            t = _timed(lambda: ops.latent_window_attention(qa, qr, cache, out, rtt, rpi, pos, *args, 0.07, **kw, **extra), reps)
+            if phase == "decode":
+                b = pairs * R * 2
+                res[f"{name}_{phase}_attention"] = dict(us=round(t * 1e6, 1), splits=kw["num_splits"], keys=per, gbs=round(b / t / 1e9), of_hbm_peak=round(b / t / HBM_PEAK, 3))
+            else:
+                fl = pairs * H * 2 * (2 * rank + rope)
+                res[f"{name}_{phase}_attention"] = dict(ms=round(t * 1e3, 3), tflops=round(fl / t / 1e12, 1), of_mfma_peak=round(fl / t / MFMA_BF16_PEAK, 3))
+        # the cache row
+        qw = H * (nope + rope)
+        a = torch.randn(n, qw + R, device=dev, generator=g).to(dt)
+        wkv = torch.ones(rank, device=dev, dtype=dt)
+        loc = torch.arange(1, n + 1, device=dev)
+        big = torch.empty(n + 8, R, device=dev, dtype=dt)
+        t = _timed(lambda: ops.latent_rows_write(a, qw, wkv, pos, loc, f, big, rank, rope, rope, True, mag, 1e-6), 20)
+        res[f"latent_rows_write_{phase}"] = dict(us=round(t * 1e6, 1), gbs=round(n * R * 2 * 2 / t / 1e9))
+        qk = s["q_rank"]
+        a2 = torch.randn(n, qk + R, device=dev, generator=g).to(dt)
+        wq = torch.ones(qk, device=dev, dtype=dt)
+        t = _timed(lambda: ops.latent_norms_rope_write(a2, wq, wkv, pos, loc, f, big, qk, rank, rope, rope, 1e-6), 20)
+        res[f"latent_norms_rope_write_{phase} (closest; norms q as well)"] = dict(us=round(t * 1e6, 1), gbs=round(n * (R + qk) * 2 * 2 / t / 1e9))
+        # W_uk per head: n x nope x rank per head
+        q3 = a[:, :qw].view(n, H, nope + rope)[..., :nope]
+        w_nk = torch.randn(H, rank, nope, device=dev, generator=g).to(dt)
+        w_kn = w_nk.transpose(1, 2).contiguous()
+        fl = 2 * n * H * nope * rank
+        byt = (n * H * (nope + rank) + H * nope * rank) * 2
+        t = _timed(lambda: torch.bmm(q3.transpose(0, 1), w_kn), 20)
+        res[f"per_head_expansion_{phase} (batched library product)"] = dict(us=round(t * 1e6, 1), tflops=round(fl / t / 1e12, 1), gbs=round(byt / t / 1e9))
+        if ops.mla_absorb_supported(n, rank, nope, 0, dt):
+            t = _timed(lambda: ops.mla_absorb(q3, w_nk), 20)
+            res[f"per_head_expansion_{phase} (one launch)"] = dict(us=round(t * 1e6, 1), tflops=round(fl / t / 1e12, 1), gbs=round(byt / t / 1e9))
+        del cache, qa, qr, out, a, a2, big
+        # the matrix memory
+        RH, dk, dv = s["rec_heads"], s["rec_dim"], s["rec_vdim"]
+        seg = {} if phase == "decode" else dict(tok_req=tok_req, seg_start=ss, seg_len=sl)
+        state = torch.zeros(nb + 1, RH, dk, dv, device=dev)
+        norm = torch.zeros(nb + 1, RH, -(-dv // ops.MATRIX_MEMORY_VALUE_BLOCK), dk + 1, device=dev)
+        r2s = torch.arange(1, nb + 1, device=dev, dtype=torch.int32)
+        p = torch.randn(n, RH * (2 * dk + 2 * dv), device=dev, generator=g).to(dt)
+        qm, km = p[:, : RH * dk].view(n, RH, dk), p[:, RH * dk: 2 * RH * dk].view(n, RH, dk)
+        vm = p[:, 2 * RH * dk: 2 * RH * dk + RH * dv].view(n, RH, dv)
+        gates = torch.randn(n, 2 * RH, device=dev, generator=g)
+        zb, fb, decay = torch.zeros(RH, device=dev), torch.full((RH,), 3.0, device=dev), torch.full((RH,), 0.97, device=dev)
+        od = torch.empty(n, RH, dv, device=dev)
+        pos = torch.full((n,), 100, device=dev, dtype=torch.int64) if phase == "decode" else pos
+        t1 = _timed(lambda: ops.matrix_memory(qm, km, vm, gates[:, :RH], gates[:, RH:], zb, fb, od, state, norm, r2s, rpi, pos, dk ** -0.5, 15.0, **seg), reps)
+        t2 = _timed(lambda: ops.linear_recurrence(qm, km, vm, od, state, r2s, rpi, pos, dk ** -0.5, head_decay=decay, **seg), reps)
+        for name, t in (("silatar_matrix_memory", t1), ("verozen_retention", t2)):
+            if phase == "decode":
+                b = n * RH * dk * dv * 4 * 2
+                res[f"{name}_decode"] = dict(us=round(t * 1e6, 1), gbs=round(b / t / 1e9), of_hbm_peak=round(b / t / HBM_PEAK, 3))
+            else:
+                res[f"{name}_prefill"] = dict(ms=round(t * 1e3, 3), vector_tflops=round(T * RH * dk * dv * 6 / t / 1e12, 2), tokens_per_s_per_sequence=round(per / t))
+    return res
+
+
+def silatar_ff_and_stream_kernels(s: dict, tokens: int) -> dict:
+    """Feed-forward and elementwise launches by the bytes or flops of their algorithm, each beside the closest model's like one."""
+    from . import ops
+    from .layers.moe import GroupedExperts
+
+    dev, dt = "cuda", torch.bfloat16
+    D, E, top, ef = s["width"], s["experts"], s["top"], s["eff"]
+    g = torch.Generator(device=dev).manual_seed(0)
+    res = {}
+
+    def put(name, t, nbytes=None, flops=None):
+        r = dict(us=round(t * 1e6, 1))
+        if nbytes:
+            r["gbs"] = round(nbytes / t / 1e9)
+        if flops:
+            r["tflops"] = round(flops / t / 1e12, 1)
+        res[name] = r
+
+    x = torch.randn(tokens, D, device=dev, generator=g)
+    y = torch.randn(tokens, D, device=dev, generator=g).to(dt)
+    w = torch.ones(D, device=dev, dtype=dt)
+    put("layernorm_residual_add", _timed(lambda: ops.layernorm_residual_add(x, y, w, w, 1e-6), 20), tokens * D * (4 + 4 + 2 + 2))
+    put("scaled_add_group_rmsnorm (closest)", _timed(lambda: ops.scaled_add_group_rmsnorm(x, y, 1.0, w, 1, 1e-6), 20), tokens * D * (4 + 4 + 2 + 2))
+    # with a token's expert rows and the gated shared branch
+    ys = torch.randn(tokens * top, D, device=dev, generator=g).to(dt)
+    rows = torch.randperm(tokens * top, device=dev, generator=g).to(torch.int32).view(tokens, top)
+    gate = torch.randn(tokens, E + 1, device=dev, generator=g)
+    put("layernorm_residual_add (expert rows, shared branch)",
+        _timed(lambda: ops.layernorm_residual_add(x, ys, w, w, 1e-6, rows=rows, y2=y, y2_gate=gate[:, E]), 20), tokens * D * (4 + 4 + 2 * (top + 1) + 2))
+    ys2 = torch.randn(tokens * (top + 1), D, device=dev, generator=g).to(dt)
+    rows2 = torch.randperm(tokens * (top + 1), device=dev, generator=g).to(torch.int32).view(tokens, top + 1)
+    coef = torch.rand(tokens, top + 1, device=dev, generator=g)
+    put("scaled_add_group_rmsnorm (expert rows; closest)",
+        _timed(lambda: ops.scaled_add_group_rmsnorm(x, ys2, 1.0, w, 1, 1e-6, rows=rows2, coef=coef), 20), tokens * D * (4 + 4 + 2 * (top + 1) + 2))
+    x.normal_(generator=g)
+    # router and gate logits
+    wr = torch.randn(E + 1, D, device=dev, generator=g).to(dt)
+    wr32 = wr[:E].float().contiguous()
+    put("project_f32 (router and shared gate)", _timed(lambda: ops.project_f32(y, wr), 20), tokens * (D * 2 + (E + 1) * 4) + wr.numel() * 2)
+    put("moe_router_logits (closest)", _timed(lambda: ops.moe_router_logits(x, wr32), 20), tokens * (D * 4 + E * 4) + wr32.numel() * 4)
+    logits = ops.project_f32(y, wr)
+    put("moe_route_scores", _timed(lambda: ops.moe_route_scores(logits[:, :E], None, top, 1, 1, 1.0, group_best=1, renorm=False), 20))
+    ids, wts = ops.moe_route_scores(logits[:, :E], None, top, 1, 1, 1.0, group_best=1, renorm=False)
+    # units between two GEMMs
+    a = torch.randn(tokens * top, 2 * ef, device=dev, generator=g).to(dt)
+    put("clamped_glu (scaled rows)", _timed(lambda: ops.clamped_glu(a, 7.0, 1.702, rows=rows, coef=wts), 20), tokens * top * ef * 2 * 3)
+    put("silu_and_mul (closest)", _timed(lambda: ops.silu_and_mul(a), 20), tokens * top * ef * 2 * 3)
+    ff = s["ff"] * 3 // 2
+    u = torch.randn(tokens, ff, device=dev, generator=g).to(dt)
+    put("activation gelu_erf", _timed(lambda: ops.activation(u, "gelu_erf"), 20), tokens * ff * 2 * 2)
+    hp = torch.randn(tokens, 2 * s["ff"], device=dev, generator=g).to(dt)
+    put("gelu_tanh_and_mul (closest)", _timed(lambda: ops.gelu_tanh_and_mul(hp[:, : s["ff"]], hp[:, s["ff"]:]), 20), tokens * s["ff"] * 2 * 3)
+    # the experts as a whole: chosen experts' weights once, or flops
+    for name, act, f_, k, wt in (("experts clamped_glu", "clamped_glu", ef, top, wts), ("experts gelu_erf (closest)", "gelu_erf", ef * 3 // 2, top, None)):
+        m = GroupedExperts(D, f_, E, dt, dev, activation=act, limit=7.0)
+        for p in (m.w_up, m.w_down):
+            p.data.normal_(0, 0.02)
+        t = _timed(lambda: m(y, ids, wt) if wt is not None else m(y, ids), 10)
+        n_used = int(ids.unique().numel())
+        put(name, t, n_used * 3 * ef * D * 2, 2 * tokens * k * 3 * ef * D)
+        del m
+    # head norm and gate of the read-out
+    RH, dv = s["rec_heads"], s["rec_vdim"]
+    o = torch.randn(tokens, RH, dv, device=dev, generator=g)
+    z = torch.randn(tokens, RH * dv, device=dev, generator=g).to(dt)
+    wh, w1 = torch.ones(RH * dv, device=dev, dtype=dt), torch.ones(dv, device=dev, dtype=dt)
+    put("head_rmsnorm_gate (weight per head)", _timed(lambda: ops.head_rmsnorm_gate_act(o, wh, z, 1e-6, dt, "sigmoid"), 20), tokens * RH * dv * (4 + 2 + 2))
+    put("head_rmsnorm_gate (shared weight; closest)", _timed(lambda: ops.head_rmsnorm_gate(o, w1, z, 1e-6, dt), 20), tokens * RH * dv * (4 + 2 + 2))
+    return res
+
+
+def run_silatar(size: str, dtype: str = "bfloat16", steps: int = 32, prefill_bs: int = 4, prefill_len: int = 2048, decode_bs: int = 64,
+                decode_ctx: int = 1024) -> dict:
+    s = SILATAR_SIZES[size]
+    if size == "sitiny":
+        prefill_bs, prefill_len, decode_bs, decode_ctx = 2, 256, 8, 128
+    out = dict(size=size, shape=s, dtype=dtype, data="synthetic", workload=dict(prefill=[prefill_bs, prefill_len], decode=[decode_bs, decode_ctx], steps=steps))
+    vz, sx = _silatar_peers(s, max(prefill_len, decode_ctx + steps + 16))
+    work = (dtype, prefill_bs, prefill_len, decode_bs, decode_ctx, steps)
+    for name, cfg in (("silatar_mixture", silatar_config(s, "mixture")), ("verozen", vz), ("silatar_latent", silatar_config(s, "latent")), ("seturax", sx)):
+        out[name] = model_throughput(cfg, *work, graph=False)
+    out["mixers"] = silatar_mixer_kernels(s, decode_bs, decode_ctx, prefill_bs, prefill_len)
+    out["ff_and_stream_decode"] = silatar_ff_and_stream_kernels(s, decode_bs)
+    out["ff_and_stream_prefill"] = silatar_ff_and_stream_kernels(s, prefill_bs * prefill_len)
+    return out
