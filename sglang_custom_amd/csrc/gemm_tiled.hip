@@ -304,23 +304,11 @@ __global__ __launch_bounds__(512) void gemm_tiled_kernel(GemmTiledParams p) {
   // two 16-byte registers per fragment slot: k-steps 0 / 1 (16-bit) or the two halves of the 32-byte
   // fp8 fragment
   i32x4 af[2][8], bf[2][4];
-#ifndef GT_ABL
-#define GT_ABL 0   // development ablations: 1 no loads in the loop, 2 no fragment reads, 3 no MFMA, 4 no vmcnt waits
-#endif
-  if (GT_ABL == 2) {
-#pragma unroll
-    for (int kk = 0; kk < 2; ++kk) {
-#pragma unroll
-      for (int mi = 0; mi < 8; ++mi) af[kk][mi] = *reinterpret_cast<const i32x4*>(sm + rd0 + mi * 2048 + kk * 64);
-#pragma unroll
-      for (int ni = 0; ni < 4; ++ni) bf[kk][ni] = *reinterpret_cast<const i32x4*>(sm + rd0 + ni * 2048 + 32768 + kk * 64);
-    }
-  }
 
 // four 1-KiB pieces of one half-tile of tile `tl`; TAIL: nothing past the last tile
 #define GT_LOAD4(ptr, ldso, tl, TAIL)                                                        \
   do {                                                                                       \
-    if (GT_ABL != 1 && (!(TAIL) || (tl) < T_)) {                                             \
+    if (!(TAIL) || (tl) < T_) {                                                              \
       char* d_ = lds_w + (((tl) & 1) ? GT_STAGE : 0) + (ldso);                               \
       _Pragma("unroll") for (int i = 0; i < 4; ++i)                                          \
           glds16(ptr[i] + (int64_t)(tl) * 128, d_ + i * 1024);                               \
@@ -338,45 +326,36 @@ __global__ __launch_bounds__(512) void gemm_tiled_kernel(GemmTiledParams p) {
     /* READ slot: request the group's two half-tiles, read the fragments of the whole K tile t */ \
     GT_LOAD4(ldA, ldA_l, (t) + 1, TAIL);                                                     \
     GT_LOAD4(ldB, ldB_l, (t) + ldB_d, TAIL);                                                 \
-    if (GT_ABL != 2) {                                                                       \
-      _Pragma("unroll") for (int kk = 0; kk < 2; ++kk) {                                     \
-        const int ro_ = rd0 ^ (FP8 ? (kk << 4) : (kk << 6));                                 \
-        const char* ab_ = sm + cur_ + a_off + ro_;                                           \
-        const char* bb_ = sm + cur_ + b_off + ro_;                                           \
-        _Pragma("unroll") for (int ni = 0; ni < 4; ++ni)                                     \
-            bf[kk][ni] = *reinterpret_cast<const i32x4*>(bb_ + ni * 2048);                   \
-        _Pragma("unroll") for (int mi = 0; mi < 8; ++mi)                                     \
-            af[kk][mi] = *reinterpret_cast<const i32x4*>(ab_ + mi * 2048);                   \
-      }                                                                                      \
+    _Pragma("unroll") for (int kk = 0; kk < 2; ++kk) {                                       \
+      const int ro_ = rd0 ^ (FP8 ? (kk << 4) : (kk << 6));                                   \
+      const char* ab_ = sm + cur_ + a_off + ro_;                                             \
+      const char* bb_ = sm + cur_ + b_off + ro_;                                             \
+      _Pragma("unroll") for (int ni = 0; ni < 4; ++ni)                                       \
+          bf[kk][ni] = *reinterpret_cast<const i32x4*>(bb_ + ni * 2048);                     \
+      _Pragma("unroll") for (int mi = 0; mi < 8; ++mi)                                       \
+          af[kk][mi] = *reinterpret_cast<const i32x4*>(ab_ + mi * 2048);                     \
     }                                                                                        \
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");                                       \
     GT_SLOT_END();                                                                           \
     /* MATRIX slot: nothing but MFMAs, then the wave's requests of its READ slot must have landed */ \
-    if (GT_ABL == 3) {                                                                       \
-      _Pragma("unroll") for (int kk = 0; kk < 2; ++kk) {                                     \
-        _Pragma("unroll") for (int mi = 0; mi < 8; ++mi) asm volatile("" ::"v"(af[kk][mi])); \
-        _Pragma("unroll") for (int ni = 0; ni < 4; ++ni) asm volatile("" ::"v"(bf[kk][ni])); \
-      }                                                                                      \
+    __builtin_amdgcn_s_setprio(1);                                                           \
+    if constexpr (FP8) {                                                                     \
+      _Pragma("unroll") for (int mi = 0; mi < 8; ++mi)                                       \
+        _Pragma("unroll") for (int ni = 0; ni < 4; ++ni) {                                   \
+          const i32x8 a8_ = __builtin_shufflevector(bf[0][ni], bf[1][ni], 0, 1, 2, 3, 4, 5, 6, 7);\
+          const i32x8 b8_ = __builtin_shufflevector(af[0][mi], af[1][mi], 0, 1, 2, 3, 4, 5, 6, 7);\
+          acc[mi][ni] = __builtin_amdgcn_mfma_scale_f32_16x16x128_f8f6f4(                    \
+              a8_, b8_, acc[mi][ni], 0, 0, 0, 0x7f7f7f7f, 0, 0x7f7f7f7f);                    \
+        }                                                                                    \
     } else {                                                                                 \
-      __builtin_amdgcn_s_setprio(1);                                                         \
-      if constexpr (FP8) {                                                                   \
+      _Pragma("unroll") for (int kk = 0; kk < 2; ++kk)                                       \
         _Pragma("unroll") for (int mi = 0; mi < 8; ++mi)                                     \
-          _Pragma("unroll") for (int ni = 0; ni < 4; ++ni) {                                 \
-            const i32x8 a8_ = __builtin_shufflevector(bf[0][ni], bf[1][ni], 0, 1, 2, 3, 4, 5, 6, 7); \
-            const i32x8 b8_ = __builtin_shufflevector(af[0][mi], af[1][mi], 0, 1, 2, 3, 4, 5, 6, 7); \
-            acc[mi][ni] = __builtin_amdgcn_mfma_scale_f32_16x16x128_f8f6f4(                  \
-                a8_, b8_, acc[mi][ni], 0, 0, 0, 0x7f7f7f7f, 0, 0x7f7f7f7f);                  \
-          }                                                                                  \
-      } else {                                                                               \
-        _Pragma("unroll") for (int kk = 0; kk < 2; ++kk)                                     \
-          _Pragma("unroll") for (int mi = 0; mi < 8; ++mi)                                   \
-            _Pragma("unroll") for (int ni = 0; ni < 4; ++ni)                                 \
-                acc[mi][ni] = Mfma<T>::run(__builtin_bit_cast(frag, bf[kk][ni]),             \
-                                           __builtin_bit_cast(frag, af[kk][mi]), acc[mi][ni]); \
-      }                                                                                      \
-      __builtin_amdgcn_s_setprio(0);                                                         \
+          _Pragma("unroll") for (int ni = 0; ni < 4; ++ni)                                   \
+              acc[mi][ni] = Mfma<T>::run(__builtin_bit_cast(frag, bf[kk][ni]),               \
+                                         __builtin_bit_cast(frag, af[kk][mi]), acc[mi][ni]); \
     }                                                                                        \
-    if (GT_ABL != 4) asm volatile("s_waitcnt vmcnt(0)" ::: "memory");                        \
+    __builtin_amdgcn_s_setprio(0);                                                           \
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");                                         \
     GT_SLOT_END();                                                                           \
   } while (0)
 
