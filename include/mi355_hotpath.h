@@ -770,7 +770,7 @@ int mi355_sigmoid_attention(void* out, const void* q, const void* k_cache, const
  *   (mi355_moe_block_rows(0), or mi355_moe_block_rows(1) for prefill-sized steps of 16-bit models) of one expert each: src_row[p] = token of sorted row p or -1 (padding), rows[pair] = p, tile_expert[block] = its expert,
  *   *n_tiles = blocks in use.  `padded` (a multiple of the block) must be at least pairs + min(experts, pairs) * (block - 1).
  * mi355_moe_grouped_linear: out[p][.] = act(weight[tile_expert[p / block]] . in[gather ? src_row[p] : p]) for every sorted
- *   row p of a block in use (0 for padding rows); weight [experts, n, k]; act = erf-GELU when `gelu`. */
+ *   row p of a block in use (0 for padding rows); weight [experts, n, k]; act: 0 nothing, 1 erf-GELU, 2 the square of relu. */
 int mi355_moe_route_grouped(int32_t* ids, float* weights, const float* logits, const float* correction, int64_t tokens,
                             int num_experts, int top, int n_groups, int keep_groups, float scale, void* stream);
 int mi355_moe_block_rows(int wide);
@@ -784,7 +784,7 @@ int mi355_moe_router_logits(float* out, const float* x, const float* weight, int
 int mi355_moe_align(int32_t* src_row, int32_t* rows, int32_t* tile_expert, int32_t* n_tiles, const int32_t* ids, int64_t tokens,
                     int top, int num_experts, int block, int64_t padded, void* stream);
 int mi355_moe_grouped_linear(void* out, const void* in, int64_t in_stride, const void* weight, const int32_t* src_row,
-                             const int32_t* tile_expert, const int32_t* n_tiles, int gather, int gelu, int64_t padded, int block,
+                             const int32_t* tile_expert, const int32_t* n_tiles, int gather, int act, int64_t padded, int block,
                              int n, int k, int dtype, void* stream);
 
 /* mi355_moe_route_scores: the same selection with its choices spelled out: score_fn 0 = sigmoid, 1 = softmax over all
@@ -983,6 +983,42 @@ int mi355_moe_route_scores_strided(int32_t* ids, float* weights, const float* lo
                                    int group_best, int renorm, void* stream);
 int mi355_clamped_glu(void* out, const void* a, int64_t a_stride, const int32_t* rows, const float* coef, int64_t pairs, int ff,
                       float limit, float alpha, int dtype, void* stream);
+
+/* ---- causal softmax attention over every earlier token, one or two score maps per head -------------------------
+ * q [tokens][heads][maps][head_dim] (a token's row contiguous), k_cache [slots][kv_heads][maps][head_dim], v_cache
+ * [slots][kv_heads][v_head_dim], out [tokens][heads][v_head_dim] (a token's row contiguous).  Per map s_j = scale * q . k_j, cap > 0:
+ * s_j <- cap * tanh(s_j / cap), a = softmax over the keys at positions 0 .. positions[t] (through the request table).
+ * maps 1: out = a_1.  maps 2: o = a_1 - lambda * a_2, out = o / sqrt(mean(o^2) + eps) * out_scale.  Then times sigmoid(gate): one
+ * logit per head (gate[t * gate_token_stride + h]) or per feature (.. + h * v_head_dim + c); gate null: nothing.
+ * runs int32 [num_runs][2] = (first token, count <= max_run) of consecutive tokens of one sequence, with tok_req [tokens]; only the
+ * listed tokens are computed.  runs null: every token alone (tok_req null: token t is sequence t).  max_run 1 takes the kernel for
+ * single tokens, whose keys may be cut into num_splits ranges (scratch fp32 num_splits * tokens * heads * maps * (v_head_dim + 2)).
+ * mi355_causal_attention_run_tokens: the longest run a launch of this shape takes. */
+int mi355_causal_attention_run_tokens(int heads, int kv_heads, int maps, int head_dim, int v_head_dim, int dtype);
+int mi355_causal_attention(void* out, const void* q, const void* k_cache, const void* v_cache, const int32_t* req_to_token,
+                           const int64_t* req_pool_indices, const int32_t* tok_req, const int64_t* positions, const int32_t* runs,
+                           int64_t num_runs, const void* gate, int gate_per_feature, int64_t gate_token_stride, int64_t q_token_stride,
+                           int64_t out_token_stride, int64_t req_to_token_stride, int heads, int kv_heads, int maps, int head_dim,
+                           int v_head_dim, float scale, float cap, float lambda, float out_scale, float eps, int num_splits,
+                           float* split_scratch, int64_t tokens, int max_run, int dtype, void* stream);
+
+/* ---- RMS norms around every sublayer of an fp32 stream, looped layers -------------------------------------------
+ * mi355_qkv_rotate_write: q [tokens][q_rows][head_dim] -> q_out (contiguous), k [tokens][k_rows][head_dim] -> k_cache row loc[t],
+ *   v [tokens][v_width] -> v_cache row loc[t]; every row of q and k divided by its root mean square if unit_norm, its first rot_dims
+ *   features rotated by positions[t] * inv_freq[i] (pairs 2 i, 2 i + 1 if interleaved, else i, i + rot_dims / 2).
+ * mi355_rmsnorm_residual_add_next: x[t] += N(b) * w_out in place, N = division by the root mean square, b = y[t] or
+ *   sum_j coef[t][j] * y[rows[t][j]] (coef null: 1); then h[t] = N(x[t]) * w_next in the activation dtype, w_next null: h[t] = x[t],
+ *   h null: nothing.
+ * mi355_pass_entry: x[t] = y[t] + table[ids[t]] + step (table [vocab][hidden] and step fp32), h[t] = N(x[t]) * w_next. */
+int mi355_qkv_rotate_write(void* q_out, void* k_cache, void* v_cache, const void* q, const void* k, const void* v, int64_t q_token_stride,
+                           int64_t k_token_stride, int64_t v_token_stride, const int64_t* positions, const int64_t* loc,
+                           const float* inv_freq, int64_t tokens, int q_rows, int k_rows, int head_dim, int v_width, int rot_dims,
+                           int interleaved, int unit_norm, float eps, int dtype, void* stream);
+int mi355_rmsnorm_residual_add_next(float* x, void* h, const void* y, int64_t y_stride, const int32_t* rows, const float* coef, int n_rows,
+                                    const void* w_out, const void* w_next, int64_t tokens, int64_t hidden, float eps, int dtype,
+                                    void* stream);
+int mi355_pass_entry(float* x, void* h, const void* y, int64_t y_stride, const float* table, const int64_t* ids, int64_t vocab,
+                     const float* step, const void* w_next, int64_t tokens, int64_t hidden, float eps, int dtype, void* stream);
 
 #ifdef __cplusplus
 }

@@ -145,6 +145,11 @@ _SIGNATURES = {
     "mi355_layernorm_residual_add": (I, [P, P, P, L, P, I, P, L, P, L, P, P, L, L, F, I, P]),
     "mi355_project_f32": (I, [P, P, L, P, L, I, I, I, P]),
     "mi355_moe_route_scores_strided": (I, [P, P, P, L, P, L, I, I, I, I, F, I, I, I, P]),
+    "mi355_causal_attention_run_tokens": (I, [I, I, I, I, I, I]),
+    "mi355_causal_attention": (I, [P, P, P, P, P, P, P, P, P, L, P, I, L, L, L, L, I, I, I, I, I, F, F, F, F, F, I, P, L, I, I, P]),
+    "mi355_qkv_rotate_write": (I, [P, P, P, P, P, P, L, L, L, P, P, P, L, I, I, I, I, I, I, I, F, I, P]),
+    "mi355_rmsnorm_residual_add_next": (I, [P, P, P, L, P, P, I, P, P, L, L, F, I, P]),
+    "mi355_pass_entry": (I, [P, P, P, L, P, P, L, P, P, L, L, F, I, P]),
     "mi355_clamped_glu": (I, [P, P, L, P, P, L, I, F, F, I, P]),
 }
 

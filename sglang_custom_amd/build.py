@@ -14,7 +14,8 @@ LIB = os.path.join(HERE, "libmi355_hotpath.so")
 LIB_DEV = os.path.join(HERE, "libmi355_hotpath_dev.so")
 SOURCES = ["elementwise.hip", "index_ops.hip", "attn_decode.hip", "attn_extend.hip", "gemm.hip",
            "gemm_tiled.hip", "sampling.hip", "quant_fp8.hip", "allreduce.hip", "mla_proj.hip",
-           "stream_ops.hip", "attn_latent.hip", "postnorm_ops.hip", "recurrence.hip", "attn_sigmoid.hip", "moe_ops.hip", "conv_ops.hip", "attn_window.hip"]
+           "stream_ops.hip", "attn_latent.hip", "postnorm_ops.hip", "recurrence.hip", "attn_sigmoid.hip", "moe_ops.hip", "conv_ops.hip", "attn_window.hip",
+           "attn_causal.hip"]
 DEV_SOURCES = ["debug_bw.hip"]
 HEADERS = [os.path.join(CSRC, "common.cuh"),
            os.path.join(os.path.dirname(HERE), "include", "mi355_hotpath.h"),
@@ -50,6 +51,8 @@ FAMILY_SOURCES = {
                 "conv_ops.hip", "attn_window.hip"],
     "Silatar": ["elementwise.hip", "index_ops.hip", "gemm.hip", "gemm_tiled.hip", "stream_ops.hip", "attn_latent.hip", "postnorm_ops.hip",
                 "recurrence.hip", "moe_ops.hip", "conv_ops.hip", "mla_proj.hip"],
+    "Lomazen": ["elementwise.hip", "index_ops.hip", "gemm.hip", "gemm_tiled.hip", "stream_ops.hip", "postnorm_ops.hip", "moe_ops.hip",
+                "attn_causal.hip"],
 }
 PARTIAL_MARK = LIB + ".partial"
 

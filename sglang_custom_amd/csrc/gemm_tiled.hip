@@ -67,7 +67,7 @@ struct GemmTiledParams {
   const int32_t* tile_expert;  // [mt] which of the stacked weight matrices tile tm uses
   const int32_t* tiles_used;   // device scalar: tiles at or past it are not computed
   int64_t w_expert_stride;     // elements between consecutive weight matrices
-  int act;                     // 1: erf-GELU on the result
+  int act;                     // on the result: 1 erf-GELU, 2 the square of relu
 };
 
 __device__ __forceinline__ void glds16(const void* g, char* l) {
@@ -433,6 +433,9 @@ __global__ __launch_bounds__(512) void gemm_tiled_kernel(GemmTiledParams p) {
               if (p.act == 1) {
                 v0 = 0.5f * v0 * (1.0f + erff(v0 * 0.7071067811865476f));
                 v1 = 0.5f * v1 * (1.0f + erff(v1 * 0.7071067811865476f));
+              } else if (p.act == 2) {
+                v0 = fmaxf(v0, 0.f); v0 *= v0;
+                v1 = fmaxf(v1, 0.f); v1 *= v1;
               }
             }
             o0.v[ni * 4 + r] = from_f32<T>(v0 + bv[ni * 4 + r]);

@@ -21,6 +21,12 @@ namespace {
 constexpr int MOE_BLOCK = 64;
 
 __device__ __forceinline__ float moe_gelu_erf(float z) { return 0.5f * z * (1.0f + erff(z * 0.7071067811865476f)); }
+// what the first grouped GEMM applies to its result: 0 nothing, 1 erf-GELU, 2 the square of relu
+__device__ __forceinline__ float moe_act(float z, int act) {
+  if (act == 1) return moe_gelu_erf(z);
+  if (act == 2) { const float r = fmaxf(z, 0.f); return r * r; }
+  return z;
+}
 
 // One wave per token; sm per wave: choice[E] | score[E] | group[G]
 __global__ __launch_bounds__(256) void moe_route_grouped_kernel(int32_t* __restrict__ ids, float* __restrict__ weights,
@@ -164,7 +170,7 @@ __global__ __launch_bounds__(256) void moe_grouped_linear_valu_kernel(T* __restr
                                                                       int64_t in_stride, const T* __restrict__ w,
                                                                       const int32_t* __restrict__ src_row,
                                                                       const int32_t* __restrict__ tile_expert,
-                                                                      const int32_t* __restrict__ n_tiles, int gather, int gelu,
+                                                                      const int32_t* __restrict__ n_tiles, int gather, int act,
                                                                       int N, int K) {
   const int tile = blockIdx.y;
   if (tile >= *n_tiles) return;
@@ -217,7 +223,7 @@ __global__ __launch_bounds__(256) void moe_grouped_linear_valu_kernel(T* __restr
       const int n = n0 + tc * 4 + j;
       if (n >= N) continue;
       float y = live ? acc[i][j] : 0.f;
-      if (gelu) y = moe_gelu_erf(y);
+      y = moe_act(y, act);
       out[(int64_t)(tile * MOE_BLOCK + r) * N + n] = from_f32<T>(y);
     }
   }
@@ -230,7 +236,7 @@ __global__ __launch_bounds__(256) void moe_grouped_linear_mfma_kernel(T* __restr
                                                                       int64_t in_stride, const T* __restrict__ w,
                                                                       const int32_t* __restrict__ src_row,
                                                                       const int32_t* __restrict__ tile_expert,
-                                                                      const int32_t* __restrict__ n_tiles, int gather, int gelu,
+                                                                      const int32_t* __restrict__ n_tiles, int gather, int act,
                                                                       int N, int K) {
   const int tile = blockIdx.y;
   if (tile >= *n_tiles) return;
@@ -284,7 +290,7 @@ __global__ __launch_bounds__(256) void moe_grouped_linear_mfma_kernel(T* __restr
       for (int r = 0; r < 4; ++r) {
         const int p = tile * MOE_BLOCK + wm * 32 + x * 16 + 4 * (lane >> 4) + r;
         float v = src_row[p] >= 0 ? acc[x][y][r] : 0.f;
-        if (gelu) v = moe_gelu_erf(v);
+        v = moe_act(v, act);
         out[(int64_t)p * N + n] = from_f32<T>(v);
       }
     }
@@ -310,7 +316,7 @@ __global__ __launch_bounds__(256) void moe_grouped_linear_wide_kernel(T* __restr
                                                                       int64_t in_stride, const T* __restrict__ w,
                                                                       const int32_t* __restrict__ src_row,
                                                                       const int32_t* __restrict__ tile_expert,
-                                                                      const int32_t* __restrict__ n_tiles, int gather, int gelu,
+                                                                      const int32_t* __restrict__ n_tiles, int gather, int act,
                                                                       int N, int K) {
   const int tile = blockIdx.y;
   if (tile >= *n_tiles) return;
@@ -399,7 +405,7 @@ __global__ __launch_bounds__(256) void moe_grouped_linear_wide_kernel(T* __restr
         const int n = n0 + wn * 64 + y * 16 + li;
         if (n >= N) continue;
         float v = live ? acc[x][y][r] : 0.f;
-        if (gelu) v = moe_gelu_erf(v);
+        v = moe_act(v, act);
         dst[n] = from_f32<T>(v);
       }
     }
@@ -520,23 +526,23 @@ __global__ void clamped_glu_kernel(T* __restrict__ out, const T* __restrict__ a,
 
 template <typename T>
 int launch_grouped(void* out, const void* in, int64_t in_stride, const void* w, const int32_t* src_row, const int32_t* tile_expert,
-                   const int32_t* n_tiles, int gather, int gelu, int N, int K, int64_t max_tiles, bool mfma, int block,
+                   const int32_t* n_tiles, int gather, int act, int N, int K, int64_t max_tiles, bool mfma, int block,
                    hipStream_t stream) {
   const dim3 grid((unsigned)cdiv(N, block), (unsigned)max_tiles);
   if constexpr (!std::is_same<T, float>::value) {
     if (mfma && block == MOE_WIDE) {
       hipLaunchKernelGGL((moe_grouped_linear_wide_kernel<T>), grid, dim3(256), 0, stream, (T*)out, (const T*)in, in_stride,
-                         (const T*)w, src_row, tile_expert, n_tiles, gather, gelu, N, K);
+                         (const T*)w, src_row, tile_expert, n_tiles, gather, act, N, K);
       return MI355_OK;
     }
     if (mfma) {
       hipLaunchKernelGGL((moe_grouped_linear_mfma_kernel<T>), grid, dim3(256), 0, stream, (T*)out, (const T*)in, in_stride,
-                         (const T*)w, src_row, tile_expert, n_tiles, gather, gelu, N, K);
+                         (const T*)w, src_row, tile_expert, n_tiles, gather, act, N, K);
       return MI355_OK;
     }
   }
   hipLaunchKernelGGL((moe_grouped_linear_valu_kernel<T>), grid, dim3(256), 0, stream, (T*)out, (const T*)in, in_stride,
-                     (const T*)w, src_row, tile_expert, n_tiles, gather, gelu, N, K);
+                     (const T*)w, src_row, tile_expert, n_tiles, gather, act, N, K);
   return MI355_OK;
 }
 
@@ -608,11 +614,12 @@ int mi355_moe_align(int32_t* src_row, int32_t* rows, int32_t* tile_expert, int32
 }
 
 int mi355_moe_grouped_linear(void* out, const void* in, int64_t in_stride, const void* weight, const int32_t* src_row,
-                             const int32_t* tile_expert, const int32_t* n_tiles, int gather, int gelu, int64_t padded, int block,
+                             const int32_t* tile_expert, const int32_t* n_tiles, int gather, int act, int64_t padded, int block,
                              int n, int k, int dtype, void* stream) {
   MI355_REQUIRE(out && in && weight && src_row && tile_expert && n_tiles, MI355_ERR_INVALID, "moe_grouped_linear: null pointer");
+  MI355_REQUIRE(act >= 0 && act <= 2, MI355_ERR_INVALID, "moe_grouped_linear: activation %d", act);
   if (block == MOE_TILED)
-    return mi355_moe_grouped_linear_tiled(out, in, in_stride, weight, gather ? src_row : nullptr, tile_expert, n_tiles, gelu ? 1 : 0,
+    return mi355_moe_grouped_linear_tiled(out, in, in_stride, weight, gather ? src_row : nullptr, tile_expert, n_tiles, act,
                                           padded, n, k, dtype, stream);
   MI355_REQUIRE(block == MOE_BLOCK || block == MOE_WIDE, MI355_ERR_INVALID, "moe_grouped_linear: blocks of %d or %d rows", MOE_BLOCK,
                 MOE_WIDE);
@@ -624,7 +631,7 @@ int mi355_moe_grouped_linear(void* out, const void* in, int64_t in_stride, const
                 "moe_grouped_linear: blocks of %d rows are for 16-bit operands with 16-byte rows", MOE_WIDE);
   int rc = MI355_OK;
   MI355_DISPATCH_DTYPE(dtype, "moe_grouped_linear", {
-    rc = launch_grouped<T>(out, in, in_stride, weight, src_row, tile_expert, n_tiles, gather, gelu, n, k, padded / block, mfma,
+    rc = launch_grouped<T>(out, in, in_stride, weight, src_row, tile_expert, n_tiles, gather, act, n, k, padded / block, mfma,
                            block, (hipStream_t)stream);
   });
   if (rc != MI355_OK) return rc;

@@ -295,6 +295,78 @@ __global__ __launch_bounds__(256) void qkv_norm_rope_write_kernel(
   }
 }
 
+// One workgroup per token: cos and sin of the token's angles once, then the rotation of its q rows (into a contiguous tensor) and
+// k rows (into the token's cache row), each row optionally divided by its root mean square (which a rotation does not change),
+// and the copy of its values into their cache row.  A row of d features belongs to `group` neighbouring lanes, V features each.
+// sm: cos [rot / 2] | sin [rot / 2]
+template <typename T, int V>
+__global__ __launch_bounds__(256) void qkv_rotate_write_kernel(
+    T* __restrict__ q_out, T* __restrict__ k_cache, T* __restrict__ v_cache, const T* __restrict__ q, const T* __restrict__ k,
+    const T* __restrict__ v, int64_t q_token_stride, int64_t k_token_stride, int64_t v_token_stride, const int64_t* __restrict__ positions,
+    const int64_t* __restrict__ loc, const float* __restrict__ inv_freq, int q_rows, int k_rows, int d, int v_width, int rot,
+    int interleaved, int unit_norm, float eps, int group) {
+  extern __shared__ __attribute__((aligned(16))) float sm[];
+  const int64_t t = blockIdx.x;
+  const int half = rot / 2, tid = threadIdx.x;
+  float* cs = sm;
+  float* sn = sm + half;
+  const float pos = (float)positions[t];
+  const int64_t slot = loc[t];
+  for (int i = tid; i < half; i += 256) sincosf(pos * inv_freq[i], &sn[i], &cs[i]);
+  for (int i = (255 - tid) * V; i < v_width; i += 256 * V)
+    stvec<T, V>(v_cache + slot * v_width + i, ldvec<T, V>(v + t * v_token_stride + i));
+  __syncthreads();
+  const int lane = tid % group, ngroups = 256 / group;
+  for (int r = tid / group; r < q_rows + k_rows; r += ngroups) {       // uniform within a row's lanes
+    const bool isq = r < q_rows;
+    const T* s = isq ? q + t * q_token_stride + (int64_t)r * d : k + t * k_token_stride + (int64_t)(r - q_rows) * d;
+    T* o = isq ? q_out + (t * q_rows + r) * (int64_t)d : k_cache + (slot * k_rows + r - q_rows) * (int64_t)d;
+    float inv = 1.0f;
+    if (unit_norm) {
+      float qs = 0.f;
+      for (int i = lane * V; i < d; i += group * V) {
+        const Vec<T, V> a = ldvec<T, V>(s + i);
+#pragma unroll
+        for (int e = 0; e < V; ++e) qs += to_f32(a.v[e]) * to_f32(a.v[e]);
+      }
+      for (int m = group >> 1; m > 0; m >>= 1) qs += __shfl_xor(qs, m, 64);
+      inv = 1.0f / sqrtf(qs / (float)d + eps);
+    }
+    for (int i = lane * V; i < d; i += group * V) {
+      const Vec<T, V> a = ldvec<T, V>(s + i);
+      Vec<T, V> w;
+      if (i >= rot) {
+#pragma unroll
+        for (int e = 0; e < V; ++e) w.v[e] = from_f32<T>(to_f32(a.v[e]) * inv);
+      } else if (interleaved) {
+#pragma unroll
+        for (int e = 0; e < V; ++e) {
+          const int f = i + e, pair = f >> 1;
+          const float x = to_f32(a.v[e]) * inv;
+          if (f >= rot) { w.v[e] = from_f32<T>(x); continue; }
+          const float y = (V > 1 ? to_f32(a.v[V > 1 ? e ^ 1 : 0]) : to_f32(s[f ^ 1])) * inv;
+          w.v[e] = from_f32<T>(f & 1 ? x * cs[pair] + y * sn[pair] : x * cs[pair] - y * sn[pair]);
+        }
+      } else {
+        Vec<T, V> p;
+        const bool whole = half % V == 0;       // then a vector's partners are a vector
+        if (whole) p = ldvec<T, V>(s + (i >= half ? i - half : i + half));
+#pragma unroll
+        for (int e = 0; e < V; ++e) {
+          const int f = i + e;
+          const float x = to_f32(a.v[e]) * inv;
+          if (f >= rot) { w.v[e] = from_f32<T>(x); continue; }
+          const bool second = f >= half;
+          const int pair = second ? f - half : f;
+          const float y = (whole ? to_f32(p.v[e]) : to_f32(s[second ? f - half : f + half])) * inv;
+          w.v[e] = from_f32<T>(second ? x * cs[pair] + y * sn[pair] : x * cs[pair] - y * sn[pair]);
+        }
+      }
+      stvec<T, V>(o + i, w);
+    }
+  }
+}
+
 // One workgroup per (token, part): out = N(y * silu(gate)) * w over one of `groups` equal consecutive parts of the row, the
 // gate applied BEFORE the norm.  y fp32 [tokens, D] contiguous, gate T row-strided, w T [D].  A part of up to 2048 features
 // keeps its gated values in registers between the two passes.
@@ -651,6 +723,33 @@ int mi355_qkv_norm_rope_write(void* q_out, void* k_cache, void* v_cache, const v
                        rot_mag);
   });
   MI355_CHECK_LAUNCH("qkv_norm_rope_write");
+  return MI355_OK;
+}
+
+int mi355_qkv_rotate_write(void* q_out, void* k_cache, void* v_cache, const void* q, const void* k, const void* v, int64_t q_token_stride,
+                           int64_t k_token_stride, int64_t v_token_stride, const int64_t* positions, const int64_t* loc,
+                           const float* inv_freq, int64_t tokens, int q_rows, int k_rows, int head_dim, int v_width, int rot_dims,
+                           int interleaved, int unit_norm, float eps, int dtype, void* stream) {
+  MI355_REQUIRE(q_out && k_cache && v_cache && q && k && v && positions && loc, MI355_ERR_INVALID, "qkv_rotate_write: null pointer");
+  MI355_REQUIRE(tokens >= 0 && tokens < (1ll << 31) && q_rows > 0 && k_rows > 0 && head_dim > 0 && head_dim <= 8192 && v_width > 0 &&
+                    q_token_stride >= (int64_t)q_rows * head_dim && k_token_stride >= (int64_t)k_rows * head_dim && v_token_stride >= v_width,
+                MI355_ERR_INVALID, "qkv_rotate_write: bad shape");
+  MI355_REQUIRE(rot_dims >= 0 && rot_dims <= head_dim && rot_dims % 2 == 0 && (rot_dims == 0 || inv_freq), MI355_ERR_INVALID,
+                "qkv_rotate_write: rot_dims must be even, at most head_dim, and come with frequencies");
+  if (tokens == 0) return MI355_OK;
+  const int vw = dtype == MI355_F32 ? 4 : 8;
+  const bool vec = head_dim % vw == 0 && v_width % vw == 0 && q_token_stride % vw == 0 && k_token_stride % vw == 0 && v_token_stride % vw == 0 &&
+                   aligned16(q_out) && aligned16(k_cache) && aligned16(v_cache) && aligned16(q) && aligned16(k) && aligned16(v);
+  int group = 1;
+  while (group < 64 && group * (vec ? vw : 1) < head_dim) group *= 2;
+  const size_t lds = (size_t)std::max(rot_dims, 2) * sizeof(float);
+  MI355_DISPATCH_DTYPE(dtype, "qkv_rotate_write", {
+    auto kern = vec ? qkv_rotate_write_kernel<T, V16<T>::n> : qkv_rotate_write_kernel<T, 1>;
+    hipLaunchKernelGGL(kern, dim3((unsigned)tokens), dim3(256), lds, (hipStream_t)stream, (T*)q_out, (T*)k_cache, (T*)v_cache, (const T*)q,
+                       (const T*)k, (const T*)v, q_token_stride, k_token_stride, v_token_stride, positions, loc, inv_freq, q_rows, k_rows,
+                       head_dim, v_width, rot_dims, interleaved, unit_norm, eps, group);
+  });
+  MI355_CHECK_LAUNCH("qkv_rotate_write");
   return MI355_OK;
 }
 

@@ -130,14 +130,16 @@ __global__ __launch_bounds__(256) void layernorm_shift_kernel(
   }
 }
 
-// One workgroup per token:  x[t] += LN(b) * w_out,  h[t] = LN(x[t]) * w_next  (w_next null: no h), with
-// b = sum_j y[rows[t][j]] (rows null: y[t]) + sigmoid(gate[t]) * y2[t] (y2 null: nothing).  KEEP > 0: the row stays in
+// One workgroup per token:  x[t] += N(b) * w_out,  h[t] = N(x[t]) * w_next  (w_next null: h[t] = x[t], h null: nothing), with
+// b = sum_j coef[t][j] * y[rows[t][j]] (coef null: 1; rows null: y[t]) + sigmoid(gate[t]) * y2[t] (y2 null: nothing); N the layer
+// norm, or (RMS) the division by the root mean square.  KEEP > 0: the row stays in
 // registers, KEEP groups of eight features per thread (D <= 2048 KEEP, 16-byte accesses); KEEP 0: any D, the row in LDS.
 struct LnAddParams {
   float* x;
   void* h;
   const void* y;
   const int32_t* rows;
+  const float* coef;
   const void* y2;
   const float* gate;
   const void* w_out;
@@ -173,9 +175,23 @@ template <typename T> __device__ __forceinline__ void st8f(T* p, const float* o)
   }
 }
 
-// (v - mean) / sqrt(var + eps) of a row held as G groups of eight per thread (groups past D hold zeros)
-template <int G>
+// (v - mean) / sqrt(var + eps), or (RMS) v / sqrt(mean v^2 + eps), of a row held as G groups of eight per thread (groups past D
+// hold zeros)
+template <int G, bool RMS>
 __device__ __forceinline__ void ln_regs(float (&v)[G][8], int64_t D, float eps, float* red) {
+  if constexpr (RMS) {
+    float q = 0.f;
+#pragma unroll
+    for (int g = 0; g < G; ++g)
+#pragma unroll
+      for (int k = 0; k < 8; ++k) q += v[g][k] * v[g][k];
+    const float inv = 1.0f / sqrtf(block_sum(q, red) / (float)D + eps);
+#pragma unroll
+    for (int g = 0; g < G; ++g)
+#pragma unroll
+      for (int k = 0; k < 8; ++k) v[g][k] *= inv;
+    return;
+  }
   float s = 0.f;
 #pragma unroll
   for (int g = 0; g < G; ++g)
@@ -201,10 +217,14 @@ __device__ __forceinline__ void ln_regs(float (&v)[G][8], int64_t D, float eps, 
 }
 
 // the same of a row in LDS, in place; every thread touches the same elements in all passes
+template <bool RMS>
 __device__ __forceinline__ void ln_lds(float* buf, int64_t D, float eps, float* red) {
-  float s = 0.f;
-  for (int64_t i = threadIdx.x; i < D; i += 256) s += buf[i];
-  const float mean = block_sum(s, red) / (float)D;
+  float mean = 0.f;
+  if constexpr (!RMS) {
+    float s = 0.f;
+    for (int64_t i = threadIdx.x; i < D; i += 256) s += buf[i];
+    mean = block_sum(s, red) / (float)D;
+  }
   float q = 0.f;
   for (int64_t i = threadIdx.x; i < D; i += 256) {
     const float d = buf[i] - mean;
@@ -214,7 +234,7 @@ __device__ __forceinline__ void ln_lds(float* buf, int64_t D, float eps, float* 
   for (int64_t i = threadIdx.x; i < D; i += 256) buf[i] = (buf[i] - mean) * inv;
 }
 
-template <typename T, int KEEP>
+template <typename T, int KEEP, bool RMS>
 __global__ __launch_bounds__(256) void layernorm_residual_add_kernel(const LnAddParams p) {
   __shared__ float red[16];
   const int64_t t = blockIdx.x, D = p.D;
@@ -239,8 +259,9 @@ __global__ __launch_bounds__(256) void layernorm_residual_add_kernel(const LnAdd
         for (int j = 0; j < p.n_rows; ++j) {      // fixed order: the sum does not depend on where the rows lie
           float e[8];
           ld8f<T>(y + (int64_t)p.rows[t * p.n_rows + j] * p.y_stride + i, e);
+          const float c = p.coef != nullptr ? p.coef[t * p.n_rows + j] : 1.0f;
 #pragma unroll
-          for (int k = 0; k < 8; ++k) v[g][k] += e[k];
+          for (int k = 0; k < 8; ++k) v[g][k] += c * e[k];
         }
       }
       if (y2 != nullptr) {
@@ -250,7 +271,7 @@ __global__ __launch_bounds__(256) void layernorm_residual_add_kernel(const LnAdd
         for (int k = 0; k < 8; ++k) v[g][k] += sg * e[k];
       }
     }
-    ln_regs<KEEP>(v, D, p.eps, red);
+    ln_regs<KEEP, RMS>(v, D, p.eps, red);
 #pragma unroll
     for (int g = 0; g < KEEP; ++g) {
       const int64_t i = 8 * ((int64_t)threadIdx.x + 256 * g);
@@ -261,9 +282,10 @@ __global__ __launch_bounds__(256) void layernorm_residual_add_kernel(const LnAdd
 #pragma unroll
       for (int k = 0; k < 8; ++k) v[g][k] = r[k] + v[g][k] * w[k];
       st8f<float>(xr + i, v[g]);
+      if (w_next == nullptr && p.h != nullptr) st8f<T>(h + i, v[g]);
     }
     if (w_next == nullptr) return;
-    ln_regs<KEEP>(v, D, p.eps, red);
+    ln_regs<KEEP, RMS>(v, D, p.eps, red);
 #pragma unroll
     for (int g = 0; g < KEEP; ++g) {
       const int64_t i = 8 * ((int64_t)threadIdx.x + 256 * g);
@@ -281,20 +303,88 @@ __global__ __launch_bounds__(256) void layernorm_residual_add_kernel(const LnAdd
       if (p.rows == nullptr) {
         b = to_f32(y[t * p.y_stride + i]);
       } else {
-        for (int j = 0; j < p.n_rows; ++j) b += to_f32(y[(int64_t)p.rows[t * p.n_rows + j] * p.y_stride + i]);
+        for (int j = 0; j < p.n_rows; ++j) {
+          const float c = p.coef != nullptr ? p.coef[t * p.n_rows + j] : 1.0f;
+          b += c * to_f32(y[(int64_t)p.rows[t * p.n_rows + j] * p.y_stride + i]);
+        }
       }
       if (y2 != nullptr) b += sg * to_f32(y2[t * p.y2_stride + i]);
       sm[i] = b;
     }
-    ln_lds(sm, D, p.eps, red);
+    ln_lds<RMS>(sm, D, p.eps, red);
     for (int64_t i = threadIdx.x; i < D; i += 256) {
       const float r = xr[i] + sm[i] * to_f32(w_out[i]);
       xr[i] = r;
       sm[i] = r;
+      if (w_next == nullptr && p.h != nullptr) h[i] = from_f32<T>(r);
     }
     if (w_next == nullptr) return;
-    ln_lds(sm, D, p.eps, red);
+    ln_lds<RMS>(sm, D, p.eps, red);
     for (int64_t i = threadIdx.x; i < D; i += 256) h[i] = from_f32<T>(sm[i] * to_f32(w_next[i]));
+  }
+}
+
+// One workgroup per token, the start of a pass over looped layers:  x[t] = y[t] + table[ids[t]] + step,  h[t] = N(x[t]) * w_next, N
+// the division by the root mean square.  KEEP as above.
+struct PassEntryParams {
+  float* x;
+  void* h;
+  const void* y;
+  const float* table;
+  const int64_t* ids;
+  const float* step;
+  const void* w_next;
+  int64_t y_stride, D, vocab;
+  float eps;
+};
+
+template <typename T, int KEEP>
+__global__ __launch_bounds__(256) void pass_entry_kernel(const PassEntryParams p) {
+  __shared__ float red[16];
+  const int64_t t = blockIdx.x, D = p.D;
+  int64_t id = p.ids[t];
+  id = id < 0 ? 0 : (id >= p.vocab ? p.vocab - 1 : id);
+  float* xr = p.x + t * D;
+  const T* y = static_cast<const T*>(p.y) + t * p.y_stride;
+  const float* tab = p.table + id * D;
+  const T* w = static_cast<const T*>(p.w_next);
+  T* h = static_cast<T*>(p.h) + t * D;
+  if constexpr (KEEP > 0) {
+    float v[KEEP][8];
+#pragma unroll
+    for (int g = 0; g < KEEP; ++g) {
+      const int64_t i = 8 * ((int64_t)threadIdx.x + 256 * g);
+#pragma unroll
+      for (int k = 0; k < 8; ++k) v[g][k] = 0.f;
+      if (i >= D) continue;
+      float e[8], s[8];
+      ld8f<T>(y + i, v[g]);
+      ld8f<float>(tab + i, e);
+      ld8f<float>(p.step + i, s);
+#pragma unroll
+      for (int k = 0; k < 8; ++k) v[g][k] += e[k] + s[k];
+      st8f<float>(xr + i, v[g]);
+    }
+    ln_regs<KEEP, true>(v, D, p.eps, red);
+#pragma unroll
+    for (int g = 0; g < KEEP; ++g) {
+      const int64_t i = 8 * ((int64_t)threadIdx.x + 256 * g);
+      if (i >= D) continue;
+      float e[8];
+      ld8f<T>(w + i, e);
+#pragma unroll
+      for (int k = 0; k < 8; ++k) e[k] *= v[g][k];
+      st8f<T>(h + i, e);
+    }
+  } else {
+    extern __shared__ __attribute__((aligned(16))) float sm[];
+    for (int64_t i = threadIdx.x; i < D; i += 256) {
+      const float r = to_f32(y[i]) + tab[i] + p.step[i];
+      xr[i] = r;
+      sm[i] = r;
+    }
+    ln_lds<true>(sm, D, p.eps, red);
+    for (int64_t i = threadIdx.x; i < D; i += 256) h[i] = from_f32<T>(sm[i] * to_f32(w[i]));
   }
 }
 
@@ -489,35 +579,73 @@ int mi355_gated_residual_add(float* x, const void* g1, const void* b1, const voi
   return MI355_OK;
 }
 
+static int norm_residual_add(LnAddParams& p, int64_t tokens, int rms, int dtype, void* stream) {
+  const int64_t hidden = p.D;
+  MI355_REQUIRE(p.x && p.y && p.w_out && (p.h != nullptr || p.w_next == nullptr), MI355_ERR_INVALID, "norm_residual_add: null pointer");
+  MI355_REQUIRE((p.y2 == nullptr) == (p.gate == nullptr) && (p.rows == nullptr || p.n_rows > 0) && (p.coef == nullptr || p.rows != nullptr),
+                MI355_ERR_INVALID, "norm_residual_add: the second branch comes with its gate, picked rows with their count, factors with rows");
+  MI355_REQUIRE(tokens >= 0 && tokens < (1ll << 31) && hidden > 0 && hidden <= 32768 && p.y_stride >= hidden &&
+                    (p.y2 == nullptr || p.y2_stride >= hidden), MI355_ERR_INVALID, "norm_residual_add: bad shape");
+  if (tokens == 0) return MI355_OK;
+  const bool vec = hidden % 8 == 0 && hidden <= 8192 && p.y_stride % 8 == 0 && aligned16(p.x) && aligned16(p.y) && aligned16(p.w_out) &&
+                   (p.h == nullptr || aligned16(p.h)) && (p.w_next == nullptr || aligned16(p.w_next)) &&
+                   (p.y2 == nullptr || (aligned16(p.y2) && p.y2_stride % 8 == 0));
+  const dim3 grid((unsigned)tokens), block(256);
+  const int keep = !vec ? 0 : hidden <= 2048 ? 1 : hidden <= 4096 ? 2 : 4;
+  const size_t lds = keep == 0 ? (size_t)hidden * sizeof(float) : 0;
+  MI355_DISPATCH_DTYPE(dtype, "norm_residual_add", {
+    auto go = [&](auto kern) {
+      if (lds > 48 * 1024) (void)hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+      hipLaunchKernelGGL(kern, grid, block, lds, (hipStream_t)stream, p);
+    };
+    switch (keep) {
+      case 1: go(rms ? layernorm_residual_add_kernel<T, 1, true> : layernorm_residual_add_kernel<T, 1, false>); break;
+      case 2: go(rms ? layernorm_residual_add_kernel<T, 2, true> : layernorm_residual_add_kernel<T, 2, false>); break;
+      case 4: go(rms ? layernorm_residual_add_kernel<T, 4, true> : layernorm_residual_add_kernel<T, 4, false>); break;
+      default: go(rms ? layernorm_residual_add_kernel<T, 0, true> : layernorm_residual_add_kernel<T, 0, false>); break;
+    }
+  });
+  MI355_CHECK_LAUNCH("norm_residual_add");
+  return MI355_OK;
+}
+
 int mi355_layernorm_residual_add(float* x, void* h, const void* y, int64_t y_stride, const int32_t* rows, int n_rows, const void* y2,
                                  int64_t y2_stride, const float* y2_gate, int64_t gate_stride, const void* w_out, const void* w_next,
                                  int64_t tokens, int64_t hidden, float eps, int dtype, void* stream) {
-  MI355_REQUIRE(x && y && w_out && (h == nullptr) == (w_next == nullptr), MI355_ERR_INVALID, "layernorm_residual_add: null pointer");
-  MI355_REQUIRE((y2 == nullptr) == (y2_gate == nullptr) && (rows == nullptr || n_rows > 0), MI355_ERR_INVALID,
-                "layernorm_residual_add: the second branch comes with its gate, picked rows with their count");
-  MI355_REQUIRE(tokens >= 0 && tokens < (1ll << 31) && hidden > 0 && hidden <= 32768 && y_stride >= hidden &&
-                    (y2 == nullptr || y2_stride >= hidden), MI355_ERR_INVALID, "layernorm_residual_add: bad shape");
-  if (tokens == 0) return MI355_OK;
+  MI355_REQUIRE((h == nullptr) == (w_next == nullptr), MI355_ERR_INVALID, "layernorm_residual_add: the next norm comes with its result");
   LnAddParams p;
-  p.x = x; p.h = h; p.y = y; p.rows = rows; p.y2 = y2; p.gate = y2_gate; p.w_out = w_out; p.w_next = w_next;
+  p.x = x; p.h = h; p.y = y; p.rows = rows; p.coef = nullptr; p.y2 = y2; p.gate = y2_gate; p.w_out = w_out; p.w_next = w_next;
   p.y_stride = y_stride; p.y2_stride = y2_stride; p.gate_stride = gate_stride; p.D = hidden; p.n_rows = n_rows; p.eps = eps;
-  const bool vec = hidden % 8 == 0 && hidden <= 8192 && y_stride % 8 == 0 && aligned16(x) && aligned16(y) && aligned16(w_out) &&
-                   (h == nullptr || (aligned16(h) && aligned16(w_next))) && (y2 == nullptr || (aligned16(y2) && y2_stride % 8 == 0));
-  const dim3 grid((unsigned)tokens), block(256);
-  MI355_DISPATCH_DTYPE(dtype, "layernorm_residual_add", {
-    if (vec && hidden <= 2048) {
-      hipLaunchKernelGGL((layernorm_residual_add_kernel<T, 1>), grid, block, 0, (hipStream_t)stream, p);
-    } else if (vec && hidden <= 4096) {
-      hipLaunchKernelGGL((layernorm_residual_add_kernel<T, 2>), grid, block, 0, (hipStream_t)stream, p);
-    } else if (vec) {
-      hipLaunchKernelGGL((layernorm_residual_add_kernel<T, 4>), grid, block, 0, (hipStream_t)stream, p);
-    } else {
-      auto kern = layernorm_residual_add_kernel<T, 0>;
-      const size_t lds = (size_t)hidden * sizeof(float);
-      if (lds > 48 * 1024) (void)hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-      hipLaunchKernelGGL(kern, grid, block, lds, (hipStream_t)stream, p);
-    }
+  return norm_residual_add(p, tokens, 0, dtype, stream);
+}
+
+int mi355_rmsnorm_residual_add_next(float* x, void* h, const void* y, int64_t y_stride, const int32_t* rows, const float* coef, int n_rows,
+                                    const void* w_out, const void* w_next, int64_t tokens, int64_t hidden, float eps, int dtype,
+                                    void* stream) {
+  LnAddParams p;
+  p.x = x; p.h = h; p.y = y; p.rows = rows; p.coef = coef; p.y2 = nullptr; p.gate = nullptr; p.w_out = w_out; p.w_next = w_next;
+  p.y_stride = y_stride; p.y2_stride = 0; p.gate_stride = 0; p.D = hidden; p.n_rows = n_rows; p.eps = eps;
+  return norm_residual_add(p, tokens, 1, dtype, stream);
+}
+
+int mi355_pass_entry(float* x, void* h, const void* y, int64_t y_stride, const float* table, const int64_t* ids, int64_t vocab,
+                     const float* step, const void* w_next, int64_t tokens, int64_t hidden, float eps, int dtype, void* stream) {
+  MI355_REQUIRE(x && h && y && table && ids && step && w_next, MI355_ERR_INVALID, "pass_entry: null pointer");
+  MI355_REQUIRE(tokens >= 0 && tokens < (1ll << 31) && hidden > 0 && hidden <= 32768 && y_stride >= hidden && vocab > 0, MI355_ERR_INVALID,
+                "pass_entry: bad shape");
+  if (tokens == 0) return MI355_OK;
+  PassEntryParams p;
+  p.x = x; p.h = h; p.y = y; p.table = table; p.ids = ids; p.step = step; p.w_next = w_next; p.y_stride = y_stride; p.D = hidden;
+  p.vocab = vocab; p.eps = eps;
+  const bool vec = hidden % 8 == 0 && hidden <= 8192 && y_stride % 8 == 0 && aligned16(x) && aligned16(y) && aligned16(h) && aligned16(table) &&
+                   aligned16(step) && aligned16(w_next);
+  const int keep = !vec ? 0 : hidden <= 2048 ? 1 : hidden <= 4096 ? 2 : 4;
+  const size_t lds = keep == 0 ? (size_t)hidden * sizeof(float) : 0;
+  MI355_DISPATCH_DTYPE(dtype, "pass_entry", {
+    auto kern = keep == 1 ? pass_entry_kernel<T, 1> : keep == 2 ? pass_entry_kernel<T, 2> : keep == 4 ? pass_entry_kernel<T, 4> : pass_entry_kernel<T, 0>;
+    if (lds > 48 * 1024) (void)hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    hipLaunchKernelGGL(kern, dim3((unsigned)tokens), dim3(256), lds, (hipStream_t)stream, p);
   });
-  MI355_CHECK_LAUNCH("layernorm_residual_add");
+  MI355_CHECK_LAUNCH("pass_entry");
   return MI355_OK;
 }

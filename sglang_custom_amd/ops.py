@@ -1555,16 +1555,17 @@ def moe_align(expert_ids: torch.Tensor, num_experts: int, wide_ok: bool = False,
     return MoePlan(src_row, rows, tile_expert, n_tiles, block, padded)
 
 
-def moe_grouped_linear(x: torch.Tensor, w: torch.Tensor, plan: MoePlan, gather: bool, gelu: bool) -> torch.Tensor:
-    """out [padded, N] = act(w[expert of the row's block] . x[src_row or the row itself]); rows of blocks not in use are
-    left unwritten (nothing reads them)."""
+def moe_grouped_linear(x: torch.Tensor, w: torch.Tensor, plan: MoePlan, gather: bool, gelu: bool, relu2: bool = False) -> torch.Tensor:
+    """out [padded, N] = act(w[expert of the row's block] . x[src_row or the row itself]), act nothing, erf-GELU or the square of
+    relu; rows of blocks not in use are left unwritten (nothing reads them)."""
+    assert not (gelu and relu2)
     _gpu(x, w)
     E, N, K = w.shape
     assert w.is_contiguous() and x.dim() == 2 and x.shape[1] == K and x.stride(1) == 1 and x.dtype == w.dtype
     assert gather or x.shape[0] == plan.padded
     out = torch.empty((plan.padded, N), dtype=x.dtype, device=x.device)
     check(_lib_().mi355_moe_grouped_linear(out.data_ptr(), x.data_ptr(), x.stride(0), w.data_ptr(), plan.src_row.data_ptr(),
-                                           plan.tile_expert.data_ptr(), plan.n_tiles.data_ptr(), int(gather), int(gelu),
+                                           plan.tile_expert.data_ptr(), plan.n_tiles.data_ptr(), int(gather), 2 if relu2 else int(gelu),
                                            plan.padded, plan.block, N, K, _dt(x), _stream(x)), "moe_grouped_linear")
     return out
 
@@ -1892,3 +1893,113 @@ def matrix_memory(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, in_logits: 
                                       blocks, q.stride(0), k.stride(0), v.stride(0), max(in_logits.stride(0), H), float(q_scale),
                                       float(gate_cap), _dt(q), _stream(q)), "matrix_memory")
     return out
+
+
+# ------------------------------------------------------- causal attention with one or two score maps, RMS norms around every sublayer
+def qkv_rotate_write(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, positions: torch.Tensor, inv_freq: torch.Tensor, rot_dims: int,
+                     interleaved: bool, unit_norm: bool, eps: float, k_cache: torch.Tensor, v_cache: torch.Tensor,
+                     loc: torch.Tensor) -> torch.Tensor:
+    """q [T, R, d], k [T, S, d] (token-strided, a token's rows contiguous), v [T, W]: rows of q and k divided by their root mean
+    square (unit_norm), their first rot_dims features rotated by position * inv_freq; q -> a new tensor, k and v -> rows loc[t] of
+    the caches [slots, ...] with S * d and W features a slot."""
+    _gpu(q, k, v, positions, inv_freq, k_cache, v_cache, loc)
+    T, R, d = q.shape
+    S, W = k.shape[1], v.shape[1]
+    assert k.shape == (T, S, d) and v.shape == (T, W) and q.dtype == k.dtype == v.dtype == k_cache.dtype == v_cache.dtype
+    assert q.stride(2) == 1 and q.stride(1) == d and k.stride(2) == 1 and k.stride(1) == d and v.stride(1) == 1
+    assert k_cache.is_contiguous() and v_cache.is_contiguous() and k_cache[0].numel() == S * d and v_cache[0].numel() == W
+    assert positions.dtype == torch.int64 and positions.numel() == T and loc.dtype == torch.int64 and loc.numel() == T
+    assert rot_dims == 0 or (inv_freq.dtype == torch.float32 and inv_freq.numel() >= rot_dims // 2 and inv_freq.is_contiguous())
+    out = torch.empty((T, R, d), dtype=q.dtype, device=q.device)
+    check(_lib_().mi355_qkv_rotate_write(out.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), q.data_ptr(), k.data_ptr(), v.data_ptr(),
+                                         max(q.stride(0), R * d), max(k.stride(0), S * d), max(v.stride(0), W), positions.data_ptr(),
+                                         loc.data_ptr(), inv_freq.data_ptr(), T, R, S, d, W, int(rot_dims), int(bool(interleaved)),
+                                         int(bool(unit_norm)), float(eps), _dt(q), _stream(q)), "qkv_rotate_write")
+    return out
+
+
+def causal_attention_run_tokens(heads: int, kv_heads: int, maps: int, head_dim: int, v_head_dim: int, dtype: torch.dtype) -> int:
+    """Most consecutive tokens of one sequence that a workgroup of causal_attention takes."""
+    return int(_lib_().mi355_causal_attention_run_tokens(heads, kv_heads, maps, head_dim, v_head_dim, _DT[dtype]))
+
+
+def causal_attention_splits(tokens: int, heads: int, kv_heads: int, max_len: Optional[int]) -> int:
+    """Key ranges per single token: about two workgroups per CU, at least 256 keys each (max_len None, a captured step: the launch
+    itself leaves ranges of shorter sequences empty)."""
+    wgs = max(1, tokens * kv_heads * ((heads // kv_heads + 15) // 16))
+    n = max(1, min(32, 512 // wgs))
+    return n if max_len is None else max(1, min(n, (max_len + 255) // 256))
+
+
+def causal_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, out: torch.Tensor, req_to_token: torch.Tensor,
+                     req_pool_indices: torch.Tensor, positions: torch.Tensor, scale: float, cap: float = 0.0, lam: float = 0.0,
+                     out_scale: float = 1.0, eps: float = 0.0, gate: Optional[torch.Tensor] = None, tok_req=None, runs=None,
+                     max_run: int = 1, num_splits: int = 1) -> torch.Tensor:
+    """q [T, H, maps, d] -> out [T, H, dv] over caches [slots, G, maps * d] / [slots, G, dv], every earlier token visible.  maps 1:
+    softmax attention, scores capped by cap (0: not).  maps 2: (map 1 - lam * map 2) over its root mean square, times out_scale.
+    gate (logits, token-strided) [T, H] or [T, H * dv]: the result times their sigmoid.  runs int32 [n, 2] of at most max_run
+    consecutive tokens of one sequence: only those tokens are computed; None: every token alone."""
+    _gpu(q, k_cache, v_cache, out, req_to_token, req_pool_indices, positions, gate, tok_req, runs)
+    T, H, maps, d = q.shape
+    G, dv = k_cache.shape[1], v_cache.shape[2]
+    assert maps in (1, 2) and H % G == 0 and k_cache.is_contiguous() and v_cache.is_contiguous()
+    assert k_cache.shape[2] == maps * d and v_cache.shape[:2] == k_cache.shape[:2] and out.shape == (T, H, dv)
+    assert q.stride(3) == 1 and q.stride(2) == d and q.stride(1) == maps * d and out.stride(2) == 1 and out.stride(1) == dv
+    assert q.dtype == out.dtype == k_cache.dtype == v_cache.dtype
+    assert req_to_token.dtype == torch.int32 and req_pool_indices.dtype == torch.int64 and positions.dtype == torch.int64
+    assert positions.numel() == T and (tok_req is None or (tok_req.dtype == torch.int32 and tok_req.numel() == T))
+    per_feature = False
+    if gate is not None:
+        assert gate.dtype == q.dtype and gate.dim() == 2 and gate.shape[0] == T and gate.shape[1] in (H, H * dv) and gate.stride(1) == 1
+        per_feature = gate.shape[1] != H
+    n = T
+    if runs is not None:
+        assert runs.dtype == torch.int32 and runs.dim() == 2 and runs.shape[1] == 2 and runs.is_contiguous()
+        n = runs.shape[0]
+    else:
+        max_run = 1
+    num_splits = num_splits if max_run == 1 else 1
+    scratch = torch.empty(num_splits * T * H * maps * (dv + 2), dtype=torch.float32, device=q.device) if num_splits > 1 else None
+    check(_lib_().mi355_causal_attention(
+        out.data_ptr(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), req_to_token.data_ptr(), req_pool_indices.data_ptr(),
+        _p(tok_req), positions.data_ptr(), _p(runs), n, _p(gate), int(per_feature), gate.stride(0) if gate is not None else 0,
+        max(q.stride(0), H * maps * d), max(out.stride(0), H * dv), req_to_token.stride(0), H, G, maps, d, dv, float(scale), float(cap),
+        float(lam), float(out_scale), float(eps), int(num_splits), _p(scratch), T, int(max_run), _dt(q), _stream(q)), "causal_attention")
+    return out
+
+
+def rmsnorm_residual_add_next(x: torch.Tensor, y: torch.Tensor, w_out: torch.Tensor, w_next: Optional[torch.Tensor], eps: float,
+                              rows: Optional[torch.Tensor] = None, coef: Optional[torch.Tensor] = None, copy: bool = False) -> Optional[torch.Tensor]:
+    """x += N(b) * w_out in place on the fp32 rows, N the division by the root mean square, b = y [T, D] or, with rows int32 [T, n],
+    sum_j coef[t, j] * y[rows[t, j]]; returns N(x) * w_next in the weights' dtype, or without w_next x itself in it (copy), or None."""
+    _gpu(x, y, w_out, w_next, rows, coef)
+    assert x.dtype == torch.float32 and x.dim() == 2 and x.is_contiguous()
+    T, D = x.shape
+    assert y.dim() == 2 and y.shape[1] == D and y.stride(1) == 1 and y.dtype == w_out.dtype
+    for w in (w_out, w_next):
+        assert w is None or (w.dtype == y.dtype and w.numel() == D and w.is_contiguous())
+    if rows is not None:
+        assert rows.dtype == torch.int32 and rows.dim() == 2 and rows.shape[0] == T and rows.is_contiguous()
+        assert coef is None or (coef.dtype == torch.float32 and coef.shape == rows.shape and coef.is_contiguous())
+    else:
+        assert y.shape[0] == T and coef is None
+    h = torch.empty((T, D), dtype=y.dtype, device=x.device) if (w_next is not None or copy) else None
+    check(_lib_().mi355_rmsnorm_residual_add_next(x.data_ptr(), _p(h), y.data_ptr(), max(y.stride(0), D), _p(rows), _p(coef),
+                                                  rows.shape[1] if rows is not None else 0, w_out.data_ptr(), _p(w_next), T, D, float(eps),
+                                                  _dt(y), _stream(x)), "rmsnorm_residual_add_next")
+    return h
+
+
+def pass_entry(x: torch.Tensor, y: torch.Tensor, table: torch.Tensor, ids: torch.Tensor, step: torch.Tensor, w_next: torch.Tensor,
+               eps: float) -> torch.Tensor:
+    """x = y + table[ids] + step in place of what the fp32 rows held; returns x over its root mean square times w_next."""
+    _gpu(x, y, table, ids, step, w_next)
+    T, D = x.shape
+    assert x.dtype == torch.float32 and x.is_contiguous() and y.shape == (T, D) and y.stride(1) == 1 and y.dtype == w_next.dtype
+    assert table.dtype == torch.float32 and table.dim() == 2 and table.shape[1] == D and table.is_contiguous()
+    assert step.dtype == torch.float32 and step.numel() == D and step.is_contiguous() and w_next.numel() == D and w_next.is_contiguous()
+    assert ids.dtype == torch.int64 and ids.numel() == T and ids.is_contiguous()
+    h = torch.empty((T, D), dtype=y.dtype, device=x.device)
+    check(_lib_().mi355_pass_entry(x.data_ptr(), h.data_ptr(), y.data_ptr(), max(y.stride(0), D), table.data_ptr(), ids.data_ptr(),
+                                   table.shape[0], step.data_ptr(), w_next.data_ptr(), T, D, float(eps), _dt(y), _stream(x)), "pass_entry")
+    return h

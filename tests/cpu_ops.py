@@ -526,7 +526,7 @@ def moe_align(expert_ids, num_experts, wide_ok=False, tiled_ok=False, block=4):
                            padded=len(src))
 
 
-def moe_grouped_linear(x, w, plan, gather, gelu):
+def moe_grouped_linear(x, w, plan, gather, gelu, relu2=False):
     out = torch.zeros((plan.padded, w.shape[1]), dtype=x.dtype)
     for p in range(plan.padded):
         r = int(plan.src_row[p])
@@ -536,6 +536,8 @@ def moe_grouped_linear(x, w, plan, gather, gelu):
         y = (x[r] if gather else x[p]).float() @ w[e].float().T
         if gelu:
             y = 0.5 * y * (1.0 + torch.erf(y * 0.7071067811865476))
+        if relu2:
+            y = torch.relu(y) ** 2
         out[p] = y.to(x.dtype)
     return out
 
@@ -777,3 +779,73 @@ def matrix_memory(q, k, v, in_logits, forget_logits, in_bias, forget_bias, out, 
             state[slot] = S
             norm_state[slot] = torch.cat([n, m[:, None]], 1)[:, None, :].expand_as(norm_state[slot])
     return out
+
+
+# ------------------------------------------------------- causal attention with one or two maps, RMS norms around every sublayer.
+# Token-by-token restatements of the header; they share nothing with oracle/lomazen_ref.py.
+def _unit(v, eps):
+    return v / torch.sqrt((v * v).mean(-1, keepdim=True) + eps)
+
+
+def qkv_rotate_write(q, k, v, positions, inv_freq, rot_dims, interleaved, unit_norm, eps, k_cache, v_cache, loc):
+    out = torch.empty_like(q, memory_format=torch.contiguous_format)
+    for t in range(q.shape[0]):
+        rows = []
+        for z in (q[t], k[t]):
+            r = _rot(z.float(), float(positions[t]), inv_freq, rot_dims, interleaved) if rot_dims else z.float()
+            rows.append(_unit(r, eps) if unit_norm else r)
+        out[t] = rows[0].to(q.dtype)
+        k_cache[int(loc[t])] = rows[1].to(k.dtype).view(k_cache.shape[1:])
+        v_cache[int(loc[t])] = v[t].view(v_cache.shape[1:])
+    return out
+
+
+def causal_attention_run_tokens(heads, kv_heads, maps, head_dim, v_head_dim, dtype):
+    return 3
+
+
+def causal_attention_splits(tokens, heads, kv_heads, max_len):
+    return 1
+
+
+def causal_attention(q, k_cache, v_cache, out, req_to_token, req_pool_indices, positions, scale, cap=0.0, lam=0.0, out_scale=1.0,
+                     eps=0.0, gate=None, tok_req=None, runs=None, max_run=1, num_splits=1):
+    T, H, maps, d = q.shape
+    G = k_cache.shape[1]
+    todo = [(t, 1) for t in range(T)] if runs is None else [(int(a), int(n)) for a, n in runs.tolist()]
+    for t0, n in todo:
+        assert n <= max_run
+        for t in range(t0, t0 + n):
+            b = t if tok_req is None else int(tok_req[t])
+            assert runs is None or int(tok_req[t0]) == b, "a run crosses two sequences"
+            slots = req_to_token[int(req_pool_indices[b]), : int(positions[t]) + 1].long()
+            kk, vv = k_cache[slots].float().view(slots.numel(), G, maps, d), v_cache[slots].float()
+            for h in range(H):
+                g = h // (H // G)
+                a = []
+                for m in range(maps):
+                    s = kk[:, g, m] @ q[t, h, m].float() * scale
+                    if cap > 0:
+                        s = cap * torch.tanh(s / cap)
+                    a.append(torch.softmax(s, 0) @ vv[:, g])
+                o = a[0] if maps == 1 else _unit(a[0] - lam * a[1], eps) * out_scale
+                if gate is not None:
+                    dv = o.numel()
+                    o = o * torch.sigmoid((gate[t, h] if gate.shape[1] == H else gate[t, h * dv: (h + 1) * dv]).float())
+                out[t, h] = o.to(out.dtype)
+    return out
+
+
+def rmsnorm_residual_add_next(x, y, w_out, w_next, eps, rows=None, coef=None, copy=False):
+    h = torch.empty_like(x)
+    for t in range(x.shape[0]):
+        b = y[t].float() if rows is None else sum((1.0 if coef is None else coef[t, j]) * y[int(r)].float() for j, r in enumerate(rows[t]))
+        x[t] += _unit(b, eps) * w_out.float()
+        h[t] = x[t] if w_next is None else _unit(x[t], eps) * w_next.float()
+    return h.to(w_out.dtype) if (w_next is not None or copy) else None
+
+
+def pass_entry(x, y, table, ids, step, w_next, eps):
+    for t in range(x.shape[0]):
+        x[t] = y[t].float() + table[int(ids[t])] + step
+    return (_unit(x, eps) * w_next.float()).to(w_next.dtype)
