@@ -35,6 +35,9 @@ class ModelConfig:
         if self.architecture == "Silatar":
             self._init_silatar(c, dtype, context_length, quantization)
             return
+        if self.architecture == "Lomazen":
+            self._init_lomazen(c, dtype, context_length, quantization)
+            return
         self.hidden_size = c["hidden_size"]
         self.num_hidden_layers = c["num_hidden_layers"]
         self.num_attention_heads = c["num_attention_heads"]
@@ -352,6 +355,70 @@ class ModelConfig:
         self.latent_kv = [(s["mixer"]["kv_rank"], s["mixer"]["rot_dim"]) if s["type"] == "latent_attention" else None for s in runs]
         self.recurrent_layer_shapes = [(s["mixer"]["heads"], s["mixer"]["dim"], s["mixer"]["vdim"]) if s["type"] == "mlstm" else None
                                        for s in runs]
+
+    def _init_lomazen(self, c: dict, dtype: str, context_length: Optional[int], quantization: Optional[str]) -> None:
+        """The Lomazen design: "layers" lists the layers one by one, {"type": "attention" | "attention_2", "mixer": {...}, "mlp":
+        {"kind": "dense", "ff"} | {"kind": "moe", "expert": {"ff"}, "router": {"experts", "top"}} | null}; widths under "width" /
+        "vocab", the norms' epsilon under "norm", the factor of the logits under "logit_scale".  Both mixers keep keys and values per
+        token (kv_layer_shapes; "attention_2" two keys per key head).  "loop" {"start", "stop", "times"}: layers start .. stop - 1 run
+        `times` times in a row with the same weights.  layer_runs lists the layer of every run, pass_starts the number of the pass
+        that begins with a run, or None; caches belong to runs, not to layers.  Layers may differ in every size."""
+        layers = c["layers"]
+        for i, spec in enumerate(layers):
+            m, mlp = spec["mixer"], spec.get("mlp")
+            if spec["type"] not in ("attention", "attention_2"):
+                raise ValueError(f"Lomazen layer {i}: unknown mixer type {spec['type']!r}")
+            if m["heads"] % m.get("kv_heads", m["heads"]):
+                raise ValueError(f"Lomazen layer {i}: {m['heads']} query heads over {m['kv_heads']} key heads")
+            if not m["scale"] > 0:
+                raise ValueError(f"Lomazen layer {i}: scale {m['scale']} is not positive")
+            rot = m.get("rot")
+            if rot and (rot.get("dims", 0) % 2 or not 0 <= rot.get("dims", 0) <= m["dim"]):
+                raise ValueError(f"Lomazen layer {i}: rotation over {rot['dims']} of {m['dim']} features")
+            if mlp is not None:
+                if mlp.get("kind") not in ("dense", "moe"):
+                    raise ValueError(f"Lomazen layer {i}: unknown feed-forward kind {mlp.get('kind')!r}")
+                if mlp["kind"] == "moe" and not 1 <= mlp["router"]["top"] <= mlp["router"]["experts"]:
+                    raise ValueError(f"Lomazen layer {i}: {mlp['router']['top']} of {mlp['router']['experts']} experts")
+        n = len(layers)
+        loop = c.get("loop")
+        a, b, times = (int(loop["start"]), int(loop["stop"]), int(loop["times"])) if loop else (0, 0, 1)
+        if not (0 <= a <= b <= n and times >= 1):
+            raise ValueError(f"Lomazen: a loop over layers {a} .. {b - 1}, {times} times, of {n} layers")
+        self.layer_runs = list(range(a)) + list(range(a, b)) * times + list(range(b, n))
+        self.loop_times = times if loop and b > a else 0
+        self.pass_starts = [None] * len(self.layer_runs)
+        for t in range(self.loop_times):
+            self.pass_starts[a + t * (b - a)] = t
+        self.layer_specs = layers
+        self.hidden_size = c["width"]
+        self.vocab_size = c["vocab"]
+        self.num_hidden_layers = len(self.layer_runs)       # what pools count: caches belong to runs
+        mixers = [s["mixer"] for s in layers]
+        self.num_attention_heads = max([m["heads"] for m in mixers] or [1])
+        self.num_key_value_heads = max([m.get("kv_heads", m["heads"]) for m in mixers] or [1])
+        self.head_dim = max([m["dim"] for m in mixers] or [1])
+        self.v_head_dim = max([m.get("vdim", m["dim"]) for m in mixers] or [1])
+        self.intermediate_size = max([s["mlp"]["ff"] if s["mlp"]["kind"] == "dense" else s["mlp"]["expert"]["ff"]
+                                      for s in layers if s.get("mlp")] or [0])
+        self.rms_norm_eps = c["norm"]["eps"]
+        self.logit_scale = float(c.get("logit_scale", 1.0))
+        self.rope_theta = None
+        self.rope_scaling = None
+        self.tie_word_embeddings = True
+        self.max_position_embeddings = context_length or 131072     # the design fixes no longest sequence
+        self.context_len = self.max_position_embeddings
+        self.quantization = quantization
+        self.dtype = _DTYPES.get(dtype) or torch.bfloat16
+        self.is_encoder_decoder = False
+        self.needs_sequence_state = False
+
+        def kv_shape(s):
+            m = s["mixer"]
+            maps = 2 if s["type"] == "attention_2" else 1
+            return (m.get("kv_heads", m["heads"]), maps * m["dim"], m.get("vdim", m["dim"]))
+
+        self.kv_layer_shapes = [kv_shape(layers[i]) for i in self.layer_runs]
 
     @classmethod
     def from_path(cls, model_path: str, **kw) -> "ModelConfig":

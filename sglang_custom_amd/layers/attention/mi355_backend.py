@@ -372,6 +372,47 @@ class Mi355AttnBackend(AttentionBackend):
             tok_req=forward_batch.token_req_index(), blocks=self._latent_blocks(forward_batch, bq), max_run=bq, num_splits=splits,
             **extra)
 
+    # ---- causal softmax attention over every earlier token, one or two score maps, per-layer key / value buffers ----
+    def _causal_runs(self, forward_batch, bq: int):
+        """(runs of two to bq consecutive tokens, single tokens) of an extend, int32 [n, 2] each on the device or None: prompts and
+        their portions take the kernel for runs, single tokens of a mixed batch the one for decode steps.  Built once per forward
+        and run length."""
+        cache = self.forward_metadata.latent_blocks
+        key = ("causal", bq)
+        if key not in cache:
+            runs, singles, t0 = [], [], 0
+            for n in forward_batch.extend_seq_lens_cpu:
+                if n == 1 or bq == 1:
+                    singles += [(t, 1) for t in range(t0, t0 + n)]
+                else:
+                    # a last token that would be a run of its own still belongs to a portion
+                    runs += [(t, min(bq, t0 + n - t)) for t in range(t0, t0 + n, bq)]
+                t0 += n
+            cache[key] = tuple(torch.tensor(r, dtype=torch.int32).to(self.device, non_blocking=True) if r else None for r in (runs, singles))
+        return cache[key]
+
+    def forward_causal(self, q, layer, forward_batch, out, cache_layer, gate=None):
+        """q [T, H, maps, d] -> out [T, H, dv].  The new tokens' keys and values are in the cache already.  A decode step, and the
+        single tokens of a mixed batch, may cut each token's keys into ranges that a second launch merges."""
+        ops = get_ops()
+        k_cache, v_cache = forward_batch.token_to_kv_pool.get_kv_buffer(cache_layer)
+        H, G = layer.tp_q_head_num, layer.tp_k_head_num
+        args = (q, k_cache, v_cache, out, forward_batch.req_to_token_pool.req_to_token, forward_batch.req_pool_indices,
+                forward_batch.positions, layer.scaling)
+        kw = dict(cap=layer.score_cap, lam=layer.map_factor, out_scale=layer.out_scale, eps=layer.eps, gate=gate)
+        longest = int(forward_batch.seq_lens_cpu.max()) if forward_batch.seq_lens_cpu is not None else None
+        if forward_batch.forward_mode.is_decode():
+            return ops.causal_attention(*args, num_splits=ops.causal_attention_splits(q.shape[0], H, G, longest), **kw)
+        tok_req = forward_batch.token_req_index()
+        bq = ops.causal_attention_run_tokens(H, G, layer.maps, layer.qk_head_dim, layer.v_head_dim, q.dtype)
+        runs, singles = self._causal_runs(forward_batch, bq)
+        if runs is not None:
+            ops.causal_attention(*args, tok_req=tok_req, runs=runs, max_run=bq, **kw)
+        if singles is not None:
+            ops.causal_attention(*args, tok_req=tok_req, runs=singles, max_run=1,
+                                 num_splits=ops.causal_attention_splits(singles.shape[0], H, G, longest), **kw)
+        return out
+
     def _windowed(self, layer) -> bool:
         """triton_backend.py:656, 711: a layer with sliding_window_size > -1 attends the window lists."""
         sw = layer.sliding_window_size

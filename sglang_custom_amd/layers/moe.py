@@ -13,6 +13,7 @@ grouped_topk / biased_grouped_topk and fused_moe_triton/layer.py FusedMoE, re-do
                       the blocks (the first gathers its rows and applies the activation in its epilogue); the weighted
                       sum over a token's experts is left to the norm kernel that consumes it
                       (GroupRMSNorm.forward(rows=, coef=)), in a fixed order.  Nothing is read back to the host.
+                      activation="relu2": the square of relu instead of the erf-GELU.
                       activation="silu_gated": down_e(silu(gate_e(h)) * up_e(h)), gate and up stacked in one weight.
                       activation="clamped_glu": the clamped gated unit (activation.ClampedGLU) instead, where a token's weight may
                       be a factor on the expert's INPUT: the projections have no bias, so it goes into the unit between them and
@@ -60,10 +61,10 @@ class GroupedTopKRouter(nn.Module):
 class GroupedExperts(nn.Module):
     def __init__(self, hidden: int, ff: int, num_experts: int, dtype, device, activation: str = "gelu_erf", limit: float = 0.0):
         super().__init__()
-        assert activation in ("gelu_erf", "silu_gated", "clamped_glu")
+        assert activation in ("gelu_erf", "relu2", "silu_gated", "clamped_glu")
         self.num_experts, self.hidden, self.ff, self.activation = num_experts, hidden, ff, activation
         # silu_gated: rows [gate (ff) | up (ff)] of every expert in one weight, as the dense models stack gate_up
-        up_rows = ff if activation == "gelu_erf" else 2 * ff
+        up_rows = ff if activation in ("gelu_erf", "relu2") else 2 * ff
         self.act = ClampedGLU(limit) if activation == "clamped_glu" else None
         self.w_up = nn.Parameter(torch.zeros(num_experts, up_rows, hidden, dtype=dtype, device=device), requires_grad=False)
         self.w_down = nn.Parameter(torch.zeros(num_experts, hidden, ff, dtype=dtype, device=device), requires_grad=False)
@@ -83,6 +84,7 @@ class GroupedExperts(nn.Module):
         elif self.activation == "silu_gated":
             a = ops.silu_and_mul(ops.moe_grouped_linear(h, self.w_up.data, plan, gather=True, gelu=False))
         else:
-            a = ops.moe_grouped_linear(h, self.w_up.data, plan, gather=True, gelu=True)
+            a = ops.moe_grouped_linear(h, self.w_up.data, plan, gather=True, gelu=self.activation == "gelu_erf",
+                                       **({"relu2": True} if self.activation == "relu2" else {}))
         y = ops.moe_grouped_linear(a, self.w_down.data, plan, gather=False, gelu=False)
         return y, plan.rows

@@ -216,6 +216,23 @@ def scaled_pair_inv_freq(base: float, dims: int, scaling: Optional[dict]):
     return torch.tensor(out, dtype=torch.float64).to(torch.float32), 0.1 * math.log(factor) + 1.0
 
 
+def banded_pair_inv_freq(base: float, dims: int, scaling: Optional[dict]) -> torch.Tensor:
+    """Frequencies of a rotation over `dims` features whose slow pairs are stretched (scaling = {"factor", "low", "high", "original"};
+    None: plain).  A pair that turns more than `high` times over `original` positions keeps its frequency, one that turns fewer
+    than `low` times has it divided by `factor`, between the two the frequency goes over linearly in the number of turns.
+    The same bands as the llama3 table of RotaryEmbedding; computed in float64 and rounded once."""
+    f = [float(base) ** (-2.0 * i / dims) for i in range(dims // 2)]
+    if scaling:
+        factor, low, high, original = (float(scaling[k]) for k in ("factor", "low", "high", "original"))
+        for i in range(len(f)):
+            turns = original * f[i] / (2.0 * math.pi)
+            if turns > high:
+                continue
+            s = 0.0 if turns < low else (turns - low) / (high - low)
+            f[i] = (1.0 - s) * f[i] / factor + s * f[i]
+    return torch.tensor(f, dtype=torch.float64).to(torch.float32)
+
+
 def pair_inv_freq(base: float, dims: int) -> torch.Tensor:
     """The same frequencies for a rotation in either pairing (feature 2 i with 2 i + 1, or i with i + dims / 2): which
     features form pair i is the kernel's business, f_i is not."""

@@ -105,4 +105,8 @@ class HipGraphRunner:
             bs, self.req_pool_indices, self.seq_lens, forward_batch.seq_lens_sum, None,
             ForwardMode.DECODE, None, forward_batch.seq_lens_cpu)
         self.graphs[bs].replay()
-        return LogitsProcessorOutput(next_token_logits=self.outputs[bs][:raw_bs])
+        out = LogitsProcessorOutput(next_token_logits=self.outputs[bs][:raw_bs])
+        rows = getattr(forward_batch, "logits_rows", None)
+        if rows is not None and rows.numel() > 0:
+            out.requested_logits = out.next_token_logits[rows]      # in a decode step token t is row t
+        return out

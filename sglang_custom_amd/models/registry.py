@@ -1,6 +1,6 @@
 """Model classes by the architecture name a configuration gives (the role of the reference's ModelRegistry,
 python/sglang/srt/models/registry.py, reduced to the families this package has).  HuggingFace configurations name
-theirs under "architectures"; Seturax, Verozen, Gatarax, Fudonex and Silatar configurations under "architecture"."""
+theirs under "architectures"; Seturax, Verozen, Gatarax, Fudonex, Silatar and Lomazen configurations under "architecture"."""
 import importlib
 
 _ARCHITECTURES = {
@@ -12,6 +12,7 @@ _ARCHITECTURES = {
     "Gatarax": ("gatarax", "GataraxForCausalLM"),
     "Fudonex": ("fudonex", "FudonexForCausalLM"),
     "Silatar": ("silatar", "SilatarForCausalLM"),
+    "Lomazen": ("lomazen", "LomazenForCausalLM"),
 }
 
 
