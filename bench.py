@@ -77,7 +77,8 @@ def parse_args():
                     help="instead of the headline workload: prefill and decode throughput of the Seturax design beside the "
                          "dense DeepSeek stack (w2048, w4096, tiny), of the Verozen design beside Llama (vz2048, vz4096, "
                          "vztiny), of the Gatarax design beside Verozen (gx2048, gx4096, gxtiny), of the Fudonex design beside Gatarax (fx2048, "
-                         "fx4096, fxtiny), or of the Silatar design beside Verozen and Seturax (si2048, si4096, sitiny), at equal layer sizes with random weights, and their hot kernels alone against the HBM / "
+                         "fx4096, fxtiny), of the Silatar design beside Verozen and Seturax (si2048, si4096, sitiny), or of the Lomazen design "
+                         "beside Llama and Verozen (lz2048, lz4096, lztiny), at equal layer sizes with random weights, and their hot kernels alone against the HBM / "
                          "matrix-core peaks; prints one JSON line (sglang_custom_amd/bench_designs.py)")
     ap.add_argument("--dry-run", action="store_true",
                     help="rendezvous rehearsal without a GPU: every rank joins a gloo group, meets at the "
@@ -318,7 +319,8 @@ def main():
         run = (bench_designs.run_verozen if args.design_compare in bench_designs.VEROZEN_SIZES else
                bench_designs.run_gatarax if args.design_compare in bench_designs.GATARAX_SIZES else
                bench_designs.run_fudonex if args.design_compare in bench_designs.FUDONEX_SIZES else
-               bench_designs.run_silatar if args.design_compare in bench_designs.SILATAR_SIZES else bench_designs.run)
+               bench_designs.run_silatar if args.design_compare in bench_designs.SILATAR_SIZES else
+               bench_designs.run_lomazen if args.design_compare in bench_designs.LOMAZEN_SIZES else bench_designs.run)
         print(json.dumps(run(args.design_compare, dtype=args.dtype, steps=args.steps)), flush=True)
         return
     if "WORLD_SIZE" not in os.environ and args.gpus > 1:

@@ -1077,3 +1077,181 @@ def run_silatar(size: str, dtype: str = "bfloat16", steps: int = 32, prefill_bs:
     out["ff_and_stream_decode"] = silatar_ff_and_stream_kernels(s, decode_bs)
     out["ff_and_stream_prefill"] = silatar_ff_and_stream_kernels(s, prefill_bs * prefill_len)
     return out
+
+
+# Lomazen's closest models: Llama for its attention (grouped heads, every earlier token, keys and values per token) and its dense
+# feed-forward, Verozen for its mixture (two matrices per expert), Silatar for its norms on both sides of a sublayer, Fudonex for
+# the launch in front of the attention.  Equal width, depth, vocabulary, heads, head widths, cache bytes per token and feed-forward
+# weights; a layer of two maps has half the heads and values twice as wide.  Lomazen's gate on the attention's result is
+# one projection more than Llama has.
+LOMAZEN_SIZES = {
+    "lz2048": dict(width=2048, heads=16, kv_heads=4, dim=128, ff=5632, experts=32, top=4, eff=1536, layers=4, vocab=32768),
+    "lz4096": dict(width=4096, heads=32, kv_heads=8, dim=128, ff=12288, experts=64, top=8, eff=1536, layers=4, vocab=32768),
+    "lztiny": dict(width=256, heads=8, kv_heads=2, dim=32, ff=512, experts=12, top=2, eff=64, layers=4, vocab=2048),
+}
+
+
+def lomazen_config(s: dict, kind: str, loop: bool = False) -> dict:
+    rot = dict(base=500000.0, dims=s["dim"], scaling=dict(factor=8.0, low=1.0, high=4.0, original=8192))
+    att = dict(type="attention", mixer=dict(heads=s["heads"], kv_heads=s["kv_heads"], dim=s["dim"], vdim=s["dim"], scale=s["dim"] ** -0.5, softcap=30.0, rot=rot))
+    two = dict(type="attention_2", mixer=dict(heads=s["heads"] // 2, kv_heads=s["kv_heads"] // 2, dim=s["dim"], vdim=2 * s["dim"], scale=s["dim"] ** -0.5, diff=0.5,
+                                              rot=dict(base=500000.0, dims=s["dim"])))
+    mlp = (dict(kind="moe", router=dict(experts=s["experts"], top=s["top"]), expert=dict(ff=s["eff"])) if kind == "mixture" else dict(kind="dense", ff=s["ff"]))
+    order = [att, two, att, two]
+    cfg = dict(architecture="Lomazen", vocab=s["vocab"], width=s["width"], norm=dict(eps=1e-6), logit_scale=0.5,
+               layers=[dict(order[i % 4], mlp=mlp) for i in range(s["layers"])])
+    if loop:
+        cfg["loop"] = dict(start=1, stop=3, times=2)
+    return cfg
+
+
+def _lomazen_peers(s: dict, dtype: str):
+    vz = verozen_config(dict(s, rec_heads=s["heads"], rec_dim=64, rec_vdim=s["dim"], groups=1, keep=1, ff=s["eff"], side=0, norm_groups=1, gate_rank=64))
+    vz.pop("token_side")
+    return llama_config(dict(s, top=1), dtype), vz
+
+
+def lomazen_mixer_kernels(s: dict, bs: int, ctx: int, prefill_bs: int, prefill_len: int) -> dict:
+    """Attention launches alone, bf16, beside Llama's on the same heads.  Decode: bytes = every key and value row once per sequence.
+    Prefill: flops 2 (d + dv) per visible pair, head and map.  Then the launch that rotates, norms and writes cache rows beside
+    Fudonex's (bytes read and written)."""
+    from . import ops
+    from .layers.rotary_embedding import banded_pair_inv_freq
+
+    dev, dt = "cuda", torch.bfloat16
+    H, G, d = s["heads"], s["kv_heads"], s["dim"]
+    g = torch.Generator(device=dev).manual_seed(0)
+    f = banded_pair_inv_freq(500000.0, d, None).to(dev)
+    res = {}
+    for phase, n, nb, per, reps in (("decode", bs, bs, ctx, 50), ("prefill", prefill_bs * prefill_len, prefill_bs, prefill_len, 20)):
+        kc = torch.randn(nb * per + 8, G, d, device=dev, generator=g).to(dt)
+        vc = torch.randn(nb * per + 8, G, d, device=dev, generator=g).to(dt)
+        k2, v2 = kc.view(-1, G // 2, 2 * d), vc.view(-1, G // 2, 2 * d)
+        rtt = (torch.arange(nb * per, device=dev, dtype=torch.int32) + 1).view(nb, per)
+        rpi = torch.arange(nb, device=dev)
+        q = torch.randn(n, H, d, device=dev, generator=g).to(dt)
+        out, out2 = torch.empty_like(q), torch.empty(n, H // 2, 2 * d, device=dev, dtype=dt)
+        gate = torch.randn(n, H * d, device=dev, generator=g).to(dt)
+        pos = torch.full((n,), per - 1, device=dev, dtype=torch.int64) if phase == "decode" else torch.arange(per, device=dev).repeat(nb)
+        tok_req = torch.repeat_interleave(torch.arange(nb, device=dev, dtype=torch.int32), per) if phase == "prefill" else None
+        pairs = nb * per if phase == "decode" else nb * per * (per + 1) // 2
+
+        def mine(maps, cap, gt):
+            HH, GG = (H, G) if maps == 1 else (H // 2, G // 2)
+            if phase == "decode":
+                kw = dict(num_splits=ops.causal_attention_splits(n, HH, GG, per))
+            else:
+                bq = ops.causal_attention_run_tokens(HH, GG, maps, d, d * maps, dt)
+                runs = [[i * per + t, min(bq, per - t)] for i in range(nb) for t in range(0, per, bq)]
+                kw = dict(tok_req=tok_req, runs=torch.tensor(runs, dtype=torch.int32, device=dev), max_run=bq)
+            qq = q.view(n, HH, maps, d)
+            kk, vv, oo = (kc, vc, out) if maps == 1 else (k2, v2, out2)
+            return (lambda: ops.causal_attention(qq, kk, vv, oo, rtt, rpi, pos, d ** -0.5, cap=cap, lam=0.4, out_scale=0.5, eps=1e-6, gate=gt, **kw)), kw.get("num_splits")
+
+        runs_ = {"lomazen one map": mine(1, 0.0, None), "lomazen one map, cap and gate": mine(1, 30.0, gate), "lomazen two maps, gate": mine(2, 0.0, gate[:, : H // 2])}
+        if phase == "decode":
+            seq = torch.full((bs,), ctx, device=dev, dtype=torch.int64)
+            nsp = int(ops.decode_num_splits(bs, G, ctx, 64))
+            logits = torch.empty(bs * H * nsp * d, device=dev, dtype=torch.float32) if nsp > 1 else None
+            lse = torch.empty(bs * H * nsp, device=dev, dtype=torch.float32) if nsp > 1 else None
+            runs_["llama"] = (lambda: ops.decode_attention_paged(q, kc, vc, out, rtt, rpi, seq, logits, lse, nsp, d ** -0.5)), nsp
+        else:
+            qo = torch.arange(0, n + 1, per, device=dev, dtype=torch.int32)
+            zero = torch.zeros(nb + 1, device=dev, dtype=torch.int32)
+            runs_["llama"] = (lambda: ops.extend_attention_fwd(q, kc[:n], vc[:n], out, kc, vc, qo, zero, zero[:1], None, True, None, per, d ** -0.5, 0.0)), None
+        for name, (fn, sp) in runs_.items():
+            t = _timed(fn, reps, warmup=reps)
+            two = "two maps" in name
+            if phase == "decode":
+                b = pairs * G * d * 2 * 2
+                res[f"{phase} attention: {name}"] = dict(us=round(t * 1e6, 1), splits=sp, gbs=round(b / t / 1e9), of_hbm_peak=round(b / t / HBM_PEAK, 3))
+            else:
+                fl = pairs * (H * 2 * 2 * d if not two else H // 2 * 2 * 2 * (d + 2 * d))
+                res[f"{phase} attention: {name}"] = dict(ms=round(t * 1e3, 3), tflops=round(fl / t / 1e12, 1), of_mfma_peak=round(fl / t / MFMA_BF16_PEAK, 3))
+        # the launch in front of it
+        p = torch.randn(n, (H + 2 * G) * d, device=dev, generator=g).to(dt)
+        loc = torch.arange(1, n + 1, device=dev)
+        w = torch.ones(d, device=dev, dtype=dt)
+        a, b_ = H * d, (H + G) * d
+        nbytes = n * (H + 2 * G) * d * 2 * 2
+        for name, fn in (("qkv_rotate_write (neighbours, unit norm)",
+                          lambda: ops.qkv_rotate_write(p[:, :a].unflatten(1, (H, d)), p[:, a:b_].unflatten(1, (G, d)), p[:, b_:], pos, f, d, True, True, 1e-6, kc, vc, loc)),
+                         ("qkv_rotate_write (halves, no norm)",
+                          lambda: ops.qkv_rotate_write(p[:, :a].unflatten(1, (H, d)), p[:, a:b_].unflatten(1, (G, d)), p[:, b_:], pos, f, d, False, False, 1e-6, kc, vc, loc)),
+                         ("qkv_norm_rope_write (closest)",
+                          lambda: ops.qkv_norm_rope_write(p[:, :a].unflatten(1, (H, d)), p[:, a:b_].unflatten(1, (G, d)), p[:, b_:].unflatten(1, (G, d)), w, w, 1e-6, pos,
+                                                          f, d, True, 1.0, kc, vc, loc))):
+            t = _timed(fn, 20, warmup=10)
+            res[f"{phase} {name}"] = dict(us=round(t * 1e6, 1), gbs=round(nbytes / t / 1e9))
+        del kc, vc, q, out, out2, gate, p
+    return res
+
+
+def lomazen_ff_and_stream_kernels(s: dict, tokens: int) -> dict:
+    """Feed-forward and elementwise launches by the bytes or flops of their algorithm, each beside the closest model's like one."""
+    from . import ops
+    from .layers.moe import GroupedExperts
+
+    dev, dt = "cuda", torch.bfloat16
+    D, E, top, ef, V = s["width"], s["experts"], s["top"], s["eff"], s["vocab"]
+    g = torch.Generator(device=dev).manual_seed(0)
+    res = {}
+
+    def put(name, fn, nbytes=None, flops=None):
+        t = _timed(fn, 20, warmup=10)
+        r = dict(us=round(t * 1e6, 1))
+        if nbytes:
+            r["gbs"] = round(nbytes / t / 1e9)
+        if flops:
+            r["tflops"] = round(flops / t / 1e12, 1)
+        res[name] = r
+
+    x = torch.randn(tokens, D, device=dev, generator=g)
+    y = torch.randn(tokens, D, device=dev, generator=g).to(dt)
+    w = torch.ones(D, device=dev, dtype=dt)
+    put("rmsnorm_residual_add_next", lambda: ops.rmsnorm_residual_add_next(x, y, w, w, 1e-6), tokens * D * (4 + 4 + 2 + 2))
+    put("layernorm_residual_add (closest)", lambda: ops.layernorm_residual_add(x, y, w, w, 1e-6), tokens * D * (4 + 4 + 2 + 2))
+    ys = torch.randn(tokens * top, D, device=dev, generator=g).to(dt)
+    rows = torch.randperm(tokens * top, device=dev, generator=g).to(torch.int32).view(tokens, top)
+    coef = torch.rand(tokens, top, device=dev, generator=g)
+    put("rmsnorm_residual_add_next (expert rows)", lambda: ops.rmsnorm_residual_add_next(x, ys, w, w, 1e-6, rows=rows, coef=coef), tokens * D * (4 + 4 + 2 * top + 2))
+    put("scaled_add_group_rmsnorm (expert rows; closest)", lambda: ops.scaled_add_group_rmsnorm(x, ys, 1.0, w, 1, 1e-6, rows=rows, coef=coef),
+        tokens * D * (4 + 4 + 2 * top + 2))
+    table, step = torch.randn(V, D, device=dev, generator=g), torch.randn(D, device=dev, generator=g)
+    ids = torch.randint(0, V, (tokens,), device=dev, generator=g)
+    put("pass_entry", lambda: ops.pass_entry(x, y, table, ids, step, w, 1e-6), tokens * D * (4 + 4 + 2 + 2))
+    x.normal_(generator=g)
+    wr = torch.randn(E, D, device=dev, generator=g).to(dt)
+    put("project_f32 (router; Silatar's)", lambda: ops.project_f32(y, wr), tokens * (D * 2 + E * 4) + wr.numel() * 2)
+    logits = ops.project_f32(y, wr)
+    put("moe_route_scores (softmax)", lambda: ops.moe_route_scores(logits, None, top, 1, 1, 1.0, score_fn="softmax", group_best=1, renorm=False))
+    put("moe_route_scores (sigmoid; closest)", lambda: ops.moe_route_scores(logits, None, top, 1, 1, 1.0, group_best=1, renorm=False))
+    ids_, _ = ops.moe_route_scores(logits, None, top, 1, 1, 1.0, score_fn="softmax", group_best=1, renorm=False)
+    for name, act in (("experts relu2", "relu2"), ("experts gelu_erf (closest)", "gelu_erf")):
+        m = GroupedExperts(D, ef, E, dt, dev, activation=act)
+        for p in (m.w_up, m.w_down):
+            p.data.normal_(0, 0.02)
+        put(name, lambda: m(y, ids_), int(ids_.unique().numel()) * 2 * ef * D * 2, 2 * tokens * top * 2 * ef * D)
+        del m
+    gu = torch.randn(tokens, 2 * s["ff"], device=dev, generator=g).to(dt)
+    put("gelu_tanh_and_mul", lambda: ops.gelu_tanh_and_mul(gu[:, : s["ff"]], gu[:, s["ff"]:]), tokens * s["ff"] * 2 * 3)
+    put("silu_and_mul (closest)", lambda: ops.silu_and_mul(gu), tokens * s["ff"] * 2 * 3)
+    return res
+
+
+def run_lomazen(size: str, dtype: str = "bfloat16", steps: int = 32, prefill_bs: int = 4, prefill_len: int = 2048, decode_bs: int = 64,
+                decode_ctx: int = 1024) -> dict:
+    s = LOMAZEN_SIZES[size]
+    if size == "lztiny":
+        prefill_bs, prefill_len, decode_bs, decode_ctx = 2, 256, 8, 128
+    out = dict(size=size, shape=s, dtype=dtype, data="synthetic", workload=dict(prefill=[prefill_bs, prefill_len], decode=[decode_bs, decode_ctx], steps=steps))
+    ll, vz = _lomazen_peers(s, dtype)
+    work = (dtype, prefill_bs, prefill_len, decode_bs, decode_ctx, steps)
+    for name, cfg, graph in (("lomazen_dense", lomazen_config(s, "dense"), True), ("llama", ll, True), ("lomazen_mixture", lomazen_config(s, "mixture"), True),
+                             ("lomazen_mixture_eager", lomazen_config(s, "mixture"), False), ("verozen", vz, False),
+                             ("lomazen_dense_loop", lomazen_config(s, "dense", loop=True), True)):
+        out[name] = model_throughput(cfg, *work, graph=graph)
+    out["mixers"] = lomazen_mixer_kernels(s, decode_bs, decode_ctx, prefill_bs, prefill_len)
+    out["ff_and_stream_decode"] = lomazen_ff_and_stream_kernels(s, decode_bs)
+    out["ff_and_stream_prefill"] = lomazen_ff_and_stream_kernels(s, prefill_bs * prefill_len)
+    return out

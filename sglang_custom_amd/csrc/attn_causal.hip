@@ -232,16 +232,18 @@ __global__ __launch_bounds__(256) void causal_attention_merge_kernel(CaArgs a) {
 #pragma unroll
   for (int m = 0; m < MAPS; ++m) {
     const float* p0 = a.partial + ((t * a.heads + h) * MAPS + m) * (int64_t)(dv + 2);
-    float M = CA_NEG;
-    for (int s = 0; s < a.num_splits; ++s) M = fmaxf(M, p0[s * stride + dv]);
-    float L = 0.f;
-    for (int s = 0; s < a.num_splits; ++s) L += p0[s * stride + dv + 1] * expf(p0[s * stride + dv] - M);
-    const float inv = (m == 1 ? -a.lambda : 1.0f) * (L > 0.f ? 1.0f / L : 0.f);
+    // lane s holds range s (at most 64 of them)
+    const bool has = lane < a.num_splits;
+    const float ms = has ? p0[lane * stride + dv] : CA_NEG, ls = has ? p0[lane * stride + dv + 1] : 0.f;
+    const float w = expf(ms - wave_max(ms));
+    const float L = wave_sum(ls * w);
+    const float wn = w * (m == 1 ? -a.lambda : 1.0f) * (L > 0.f ? 1.0f / L : 0.f);
+#pragma unroll 4
     for (int s = 0; s < a.num_splits; ++s) {
-      const float f = expf(p0[s * stride + dv] - M) * inv;
+      const float f = __shfl(wn, s, 64);
 #pragma unroll
       for (int u = 0; u < 8; ++u)
-        if (lane + 64 * u < dv) o[u] += p0[s * stride + lane + 64 * u] * f;
+        if (64 * u < dv && lane + 64 * u < dv) o[u] += p0[s * stride + lane + 64 * u] * f;
     }
   }
   float mul = 1.f;
@@ -266,14 +268,19 @@ __global__ __launch_bounds__(256) void causal_attention_merge_kernel(CaArgs a) {
 // ------------------------------------------------------------------------------------------------ prompts, matrix cores
 // S^T = K Q^T (A = 32 key rows from LDS, B = the wave's 32 queries in registers), so a lane owns its query's scores, and the
 // rounded weights are the B operand of O^T += V^T P^T (A by transposed reads of the row-major V tile); see the layout notes of
-// the 32x32x16 instruction in common.cuh.  Key tiles of 64, the next tile in registers while the current one is multiplied.
+// the 32x32x16 instruction in common.cuh.  Key tiles of 64 (32 where results and queries fill the registers), the next tile in
+// registers and the cache slots of the one after it while the current one is multiplied.
 // LDS rows: K rows have an odd number of 16-byte chunks (16 consecutive rows start in 16 different bank groups), V rows a number
 // that is 4 or 12 modulo 16 (the four rows of a transposed read start 64 bytes apart).
 // KS: score steps of 16 features (d <= 16 KS, the rest zero), VT: 32-column tiles of the result (dv <= 32 VT).
 template <int KS, int MAPS> constexpr int ca_k_pitch() { return (2 * KS * MAPS + 1) * 16; }
 template <int VT> constexpr int ca_v_pitch() { return 4 * (VT | 1) * 16; }
+// keys per tile, and workgroups per CU: two where queries, results and the staged tile leave room in 256 registers
+constexpr int ca_regs(int ks, int vt, int maps, int keys) { return 4 * ks + 16 * vt + keys * (2 * ks * maps + 4 * vt) / 64 + keys / 2; }
+constexpr int ca_keys(int ks, int vt, int maps) { return ca_regs(ks, vt, maps, 64) <= 176 || ca_regs(ks, vt, maps, 32) > 208 ? 64 : 32; }
+constexpr int ca_waves(int ks, int vt, int maps) { return ca_regs(ks, vt, maps, ca_keys(ks, vt, maps)) <= 208 ? 2 : 1; }
 template <int KS, int VT, int MAPS> constexpr size_t ca_tile_lds() {
-  const size_t kv = (size_t)64 * (ca_k_pitch<KS, MAPS>() + ca_v_pitch<VT>());
+  const size_t kv = (size_t)ca_keys(KS, VT, MAPS) * (ca_k_pitch<KS, MAPS>() + ca_v_pitch<VT>());
   const size_t ex = MAPS == 2 ? (size_t)64 * (32 * VT + 4) * 4 : 0;
   return kv > ex ? kv : ex;
 }
@@ -282,10 +289,12 @@ template <typename T, int KS, int VT, int MAPS, bool CAP>
 __device__ __forceinline__ void causal_attention_tile_body(const CaArgs& a, char* sm) {
   using frag = typename Mfma32<T>::frag;
   constexpr int KP = ca_k_pitch<KS, MAPS>(), VP = ca_v_pitch<VT>();
-  constexpr int ROWS = MAPS == 2 ? 64 : 128;
-  constexpr int KN = (64 * 2 * KS * MAPS + 255) / 256, VN = (64 * 4 * VT + 255) / 256;     // 16-byte chunks per thread
+  constexpr int BN = ca_keys(KS, VT, MAPS), HF = BN / 32;      // keys per tile, in halves of 32
+  constexpr int KL = 2 * KS * MAPS, VL = 4 * VT;               // 16-byte chunks of a (padded) key and value row
+  constexpr int KN = BN * KL / 256, VN = BN * VL / 256;        // chunks per thread
+  static_assert(KN >= 1 && VN >= 1 && 256 % KL == 0 && 256 % VL == 0, "a thread's chunks lie in one column");
   char* ks = sm;
-  char* vs = sm + 64 * KP;
+  char* vs = sm + BN * KP;
   const int rep = a.heads / a.kv_heads, HR = a.rows_heads;
   const int chunks = (rep + HR - 1) / HR, per_run = a.kv_heads * chunks;
   // consecutive workgroups differ in the key head (they go round-robin over the XCDs); long, late runs first
@@ -320,53 +329,40 @@ __device__ __forceinline__ void causal_attention_tile_body(const CaArgs& a, char
       qf[s] = i < d ? v : zero;
     }
   }
-  // a map's features past d in the K tile are zeros for good (the queries' are too, but 0 * garbage may be NaN)
-  if (d < 16 * KS) {
-    const int dch = d / 8, pad = 2 * KS - dch;
-    const Vec<T, 8> zero = __builtin_bit_cast(Vec<T, 8>, lds_u32x4{0, 0, 0, 0});
-    for (int e = threadIdx.x; e < 64 * MAPS * pad; e += 256) {
-      const int r = e / (MAPS * pad), x = e - r * (MAPS * pad), m = x / pad;
-      lds_store16(ks + r * KP + 16 * (m * 2 * KS + dch + x - m * pad), zero);
-    }
-  }
-  // staging: thread -> (key row, chunk) of up to KN (VN) pieces of a tile
-  const int dch = d / 8, kch = MAPS * dch, vch = dv / 8;
-  const T* kc = (const T*)a.k_cache + (int64_t)g * MAPS * d;
-  const T* vc = (const T*)a.v_cache + (int64_t)g * dv;
+  // staging: a thread owns one chunk column of the K rows tid / KL + u * 256 / KL and of the V rows tid / VL + u * 256 / VL; a map's
+  // features past d are zeros in the K tile (the queries' are too, but 0 * garbage may be NaN), columns past dv are left alone
+  const int kr0 = threadIdx.x / KL, kch = threadIdx.x % KL, kmap = kch / (2 * KS), kc0 = (kch % (2 * KS)) * 8;
+  const int vr0 = threadIdx.x / VL, vc0 = (threadIdx.x % VL) * 8;
+  const bool klive = kc0 < d, vlive = vc0 < dv;
+  const T* kc = (const T*)a.k_cache + ((int64_t)g * MAPS + kmap) * d + (klive ? kc0 : 0);
+  const T* vc = (const T*)a.v_cache + (int64_t)g * dv + (vlive ? vc0 : 0);
   const int64_t krow = (int64_t)a.kv_heads * MAPS * d, vrow_ = (int64_t)a.kv_heads * dv;
-  int kk_[KN], ko_[KN], kl_[KN], vk_[VN], vo_[VN];
-#pragma unroll
-  for (int u = 0; u < KN; ++u) {
-    const int e = threadIdx.x + 256 * u, ec = min(e, 64 * kch - 1);
-    const int r = ec / kch, ch = ec - r * kch, m = MAPS == 2 && ch >= dch ? 1 : 0;
-    kk_[u] = r;
-    ko_[u] = ch * 8;
-    kl_[u] = e < 64 * kch ? r * KP + 16 * (m * 2 * KS + ch - m * dch) : -1;
-  }
-#pragma unroll
-  for (int u = 0; u < VN; ++u) {
-    const int e = threadIdx.x + 256 * u, ec = min(e, 64 * vch - 1);
-    const int r = ec / vch;
-    vk_[u] = e < 64 * vch ? r : -1 - r;
-    vo_[u] = (ec - r * vch) * 8;
-  }
+  char* kst = ks + kr0 * KP + 16 * kch;
+  char* vst = vs + vr0 * VP + 2 * vc0;
+  int kslot[KN], vslot[KL == VL ? 1 : VN];
   Vec<T, 8> kreg[KN], vreg[VN];
-  auto load_tile = [&](int kt) {          // unconditional loads: keys past the last one are clamped (and masked below)
+  auto load_slots = [&](int kt) {         // keys past the last one are clamped (and masked below)
 #pragma unroll
-    for (int u = 0; u < KN; ++u) kreg[u] = ldvec<T, 8>(kc + (int64_t)table[min(kt * 64 + kk_[u], last)] * krow + ko_[u]);
+    for (int u = 0; u < KN; ++u) kslot[u] = table[min(kt * BN + kr0 + u * (256 / KL), last)];
+    if constexpr (KL != VL) {
 #pragma unroll
-    for (int u = 0; u < VN; ++u) {
-      const int r = vk_[u] < 0 ? -1 - vk_[u] : vk_[u];
-      vreg[u] = ldvec<T, 8>(vc + (int64_t)table[min(kt * 64 + r, last)] * vrow_ + vo_[u]);
+      for (int u = 0; u < VN; ++u) vslot[u] = table[min(kt * BN + vr0 + u * (256 / VL), last)];
     }
   };
+  auto load_tile = [&]() {
+#pragma unroll
+    for (int u = 0; u < KN; ++u) kreg[u] = ldvec<T, 8>(kc + (int64_t)kslot[u] * krow);
+#pragma unroll
+    for (int u = 0; u < VN; ++u) vreg[u] = ldvec<T, 8>(vc + (int64_t)(KL == VL ? kslot[u % KN] : vslot[KL == VL ? 0 : u]) * vrow_);
+  };
   auto store_tile = [&]() {
+    const Vec<T, 8> zero = __builtin_bit_cast(Vec<T, 8>, lds_u32x4{0, 0, 0, 0});
 #pragma unroll
-    for (int u = 0; u < KN; ++u)
-      if (kl_[u] >= 0) lds_store16(ks + kl_[u], kreg[u]);
+    for (int u = 0; u < KN; ++u) lds_store16(kst + u * (256 / KL) * KP, klive ? kreg[u] : zero);
+    if (vlive) {
 #pragma unroll
-    for (int u = 0; u < VN; ++u)
-      if (vk_[u] >= 0) lds_store16(vs + vk_[u] * VP + 2 * vo_[u], vreg[u]);
+      for (int u = 0; u < VN; ++u) lds_store16(vst + u * (256 / VL) * VP, vreg[u]);
+    }
   };
 
   f32x16 ot[VT];
@@ -382,23 +378,30 @@ __device__ __forceinline__ void causal_attention_tile_body(const CaArgs& a, char
   auto k_frag = [&](int s, int hf) -> frag { return lds_load16<frag>(k_rd + 32 * KP * hf + 32 * s); };
   const int l16 = lane & 15, dhalf = (lane >> 4) & 1, tq = l16 >> 2, tpp = l16 & 3;
   const char* v_rd = vs + VP * (4 * hh + tq) + 32 * dhalf + 8 * tpp;
-  const int n_tiles = last / 64 + 1;
-  load_tile(0);
+  const int n_tiles = last / BN + 1;
+  load_slots(0);
+  load_tile();
+  load_slots(min(1, n_tiles - 1));
   for (int kt = 0; kt < n_tiles; ++kt) {
     __syncthreads();            // the previous tile is consumed
     store_tile();
     __syncthreads();
-    if (kt + 1 < n_tiles) load_tile(kt + 1);
-    if (wave_idle || kt * 64 > wave_max_limit) continue;      // nothing of this tile is seen by this wave (wave-uniform)
-    f32x16 st[2];
+    if (kt + 1 < n_tiles) {
+      load_tile();
+      load_slots(min(kt + 2, n_tiles - 1));
+    }
+    if (wave_idle || kt * BN > wave_max_limit) continue;      // nothing of this tile is seen by this wave (wave-uniform)
+    f32x16 st[HF];
 #pragma unroll
-    for (int hf = 0; hf < 2; ++hf)
+    for (int hf = 0; hf < HF; ++hf)
 #pragma unroll
       for (int i = 0; i < 16; ++i) st[hf][i] = 0.f;
     // fragments are read two steps ahead of the products that use them
-    frag kr[3][2];
+    frag kr[3][HF];
 #pragma unroll
-    for (int s = 0; s < 2 && s < KS; ++s) { kr[s][0] = k_frag(s, 0); kr[s][1] = k_frag(s, 1); }
+    for (int s = 0; s < 2; ++s)
+#pragma unroll
+      for (int hf = 0; hf < HF; ++hf) kr[s][hf] = k_frag(s, hf);
     typename TrRead<T>::v4 vlo[4], vhi[4];                    // ring of four (16-key step, column tile) fragments
     auto v_read = [&](int i, int slot) {
       const int u = i / VT, c = i % VT;
@@ -409,8 +412,8 @@ __device__ __forceinline__ void causal_attention_tile_body(const CaArgs& a, char
 #pragma unroll
     for (int s = 0; s < KS; ++s) {
       if (s + 2 < KS) {
-        kr[(s + 2) % 3][0] = k_frag(s + 2, 0);
-        kr[(s + 2) % 3][1] = k_frag(s + 2, 1);
+#pragma unroll
+        for (int hf = 0; hf < HF; ++hf) kr[(s + 2) % 3][hf] = k_frag(s + 2, hf);
       } else if (s == KS - 2) {
         v_read(0, 0);
         v_read(1, 1);
@@ -419,21 +422,21 @@ __device__ __forceinline__ void causal_attention_tile_body(const CaArgs& a, char
         v_read(3, 3);
       }
       __builtin_amdgcn_sched_barrier(0);
-      st[0] = Mfma32<T>::run(kr[s % 3][0], qf[s], st[0]);
-      st[1] = Mfma32<T>::run(kr[s % 3][1], qf[s], st[1]);
+#pragma unroll
+      for (int hf = 0; hf < HF; ++hf) st[hf] = Mfma32<T>::run(kr[s % 3][hf], qf[s], st[hf]);
       __builtin_amdgcn_sched_barrier(0);
     }
     if constexpr (CAP) {
 #pragma unroll
-      for (int hf = 0; hf < 2; ++hf)
+      for (int hf = 0; hf < HF; ++hf)
 #pragma unroll
         for (int i = 0; i < 16; ++i) st[hf][i] = ca_cap_fast(st[hf][i], a.cap, k2);
     }
     float mloc = -INFINITY;
-    if (kt * 64 + 63 > wave_min_limit) {                      // only tiles that cross the wave's diagonal are masked
-      const int lim = my_limit - kt * 64 - 4 * hh;
+    if (kt * BN + BN - 1 > wave_min_limit) {                      // only tiles that cross the wave's diagonal are masked
+      const int lim = my_limit - kt * BN - 4 * hh;
 #pragma unroll
-      for (int hf = 0; hf < 2; ++hf)
+      for (int hf = 0; hf < HF; ++hf)
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
           const float x = (32 * hf + 8 * (i >> 2) + (i & 3)) > lim ? -INFINITY : st[hf][i];
@@ -442,7 +445,7 @@ __device__ __forceinline__ void causal_attention_tile_body(const CaArgs& a, char
         }
     } else {
 #pragma unroll
-      for (int hf = 0; hf < 2; ++hf)
+      for (int hf = 0; hf < HF; ++hf)
 #pragma unroll
         for (int i = 0; i < 16; ++i) mloc = fmaxf(mloc, st[hf][i]);
     }
@@ -452,9 +455,9 @@ __device__ __forceinline__ void causal_attention_tile_body(const CaArgs& a, char
     const float alpha = __builtin_amdgcn_exp2f(m - ms);
     m = mnew;
     float psum = 0.f;
-    frag pb[4];
+    frag pb[2 * HF];
 #pragma unroll
-    for (int hf = 0; hf < 2; ++hf)
+    for (int hf = 0; hf < HF; ++hf)
 #pragma unroll
       for (int i = 0; i < 16; ++i) {
         const float pe = __builtin_amdgcn_exp2f(__builtin_fmaf(st[hf][i], qmul, -ms));
@@ -468,7 +471,7 @@ __device__ __forceinline__ void causal_attention_tile_body(const CaArgs& a, char
     }
     __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-    for (int i = 0; i < 4 * VT; ++i) {                        // fragment i + 4 is requested right behind product i
+    for (int i = 0; i < 2 * HF * VT; ++i) {                        // fragment i + 4 is requested right behind product i
       frag va;
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
@@ -477,7 +480,7 @@ __device__ __forceinline__ void causal_attention_tile_body(const CaArgs& a, char
       }
       ot[i % VT] = Mfma32<T>::run(va, pb[i / VT], ot[i % VT]);
       __builtin_amdgcn_sched_barrier(0);
-      if (i + 4 < 4 * VT) {
+      if (i + 4 < 2 * HF * VT) {
         v_read(i + 4, i & 3);
         __builtin_amdgcn_sched_barrier(0);
       }
@@ -546,34 +549,34 @@ __device__ __forceinline__ void causal_attention_tile_body(const CaArgs& a, char
     }
 }
 
-// two workgroups per CU where queries, results and the staged tile leave room in 256 registers
-constexpr int ca_tile_waves(int ks, int vt, int maps) { return 4 * ks + 20 * vt + 2 * ks * maps <= 136 ? 2 : 1; }
 template <typename T, int KS, int VT, int MAPS, bool CAP>
-__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(ca_tile_waves(KS, VT, MAPS), ca_tile_waves(KS, VT, MAPS))))
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(ca_waves(KS, VT, MAPS), ca_waves(KS, VT, MAPS))))
 void causal_attention_tile_kernel(CaArgs a) {
   extern __shared__ __attribute__((aligned(16))) char smt[];
   causal_attention_tile_body<T, KS, VT, MAPS, CAP>(a, smt);
 }
 
 // ------------------------------------------------------------------------------------------------ single tokens, matrix cores
-// A workgroup: one token, one key head, up to 16 of its query heads, one range of the token's keys.  Wave w takes the key tiles
-// (32 keys) w, w + 4, ... of the range, each on its own: S = K Q^T puts head l & 15 and keys 4 (l >> 4) + r of two 16-key halves
-// into lane l; the rounded weights are the B operand of O^T += V^T P^T with the keys in just that order; V goes through a
+// A workgroup: one token, one key head, up to 16 of its query heads, one range of the token's keys.  A wave takes key tiles (32 keys)
+// of the range on its own: one map, every fourth tile; two maps, waves 0 and 2 the first map and 1 and 3 the second, every second
+// tile (the pair's second reading of the values comes from L2).  S = K Q^T puts head l & 15 and keys 4 (l >> 4) + r of two 16-key
+// halves into lane l; the rounded weights are the B operand of O^T += V^T P^T with the keys in just that order; V goes through a
 // wave-private piece of LDS for the transposed reads.  The waves' results meet in LDS at the end.
 // KS: score steps of 32 features (d <= 32 KS, the rest zero), VC: 16-column tiles of the result (dv <= 16 VC).
 template <int VC> constexpr int ct_v_pitch() { return 4 * (((VC + 1) / 2) | 1) * 16; }
-template <int VC, int MAPS> constexpr size_t ct_lds() {
-  const size_t v = (size_t)4 * 32 * ct_v_pitch<VC>(), ex = (size_t)2 * MAPS * 16 * (16 * VC + 4) * 4;
+template <int VC> constexpr size_t ct_lds() {
+  const size_t v = (size_t)4 * 32 * ct_v_pitch<VC>(), ex = (size_t)2 * 16 * (16 * VC + 4) * 4;
   return v > ex ? v : ex;
 }
 
 template <typename T, int KS, int VC, int MAPS>
 __global__ __launch_bounds__(256) void causal_attention_token_kernel(CaArgs a) {
   extern __shared__ __attribute__((aligned(16))) char smd[];
-  __shared__ float red_m[4][MAPS][16], red_l[4][MAPS][16];
+  __shared__ float red_m[4][16], red_l[4][16];
   using frag = typename Mfma<T>::frag;
   constexpr int VP = ct_v_pitch<VC>();
-  constexpr int VN = VC;                      // 16-byte chunks of a V tile per lane: 32 rows x 2 VC chunks over 64 lanes
+  constexpr int VL = 2 * VC, VN = VC;         // 16-byte chunks of a (padded) value row; chunks of a V tile per lane
+  constexpr int STREAMS = 4 / MAPS;           // waves that walk the range side by side
   const int rep = a.heads / a.kv_heads;
   const int chunks = (rep + 15) / 16, per_run = a.kv_heads * chunks;
   const int64_t run = blockIdx.x / per_run;
@@ -582,7 +585,8 @@ __global__ __launch_bounds__(256) void causal_attention_token_kernel(CaArgs a) {
   const int b = a.tok_req != nullptr ? a.tok_req[t] : (int)t;
   const int32_t* table = a.req_to_token + a.req_pool_indices[b] * a.req_to_token_stride;
   const int h0 = g * rep + hc * 16, nh = min(16, rep - hc * 16);
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int map = MAPS == 2 ? wave & 1 : 0, stream = MAPS == 2 ? wave >> 1 : wave;
   const int li = lane & 15, lg = lane >> 4;
   const int d = a.d, dv = a.dv;
   const int len = (int)a.positions[t] + 1;
@@ -591,44 +595,33 @@ __global__ __launch_bounds__(256) void causal_attention_token_kernel(CaArgs a) {
   const int per = max((ntiles + a.num_splits - 1) / a.num_splits, a.num_splits > 1 ? min(8, ntiles) : 1);
   const int split = blockIdx.y;
   const int tile_lo = split * per, tile_hi = min(ntiles, tile_lo + per);
-  const T* kc = (const T*)a.k_cache + (int64_t)g * MAPS * d;
-  const T* vc = (const T*)a.v_cache + (int64_t)g * dv;
+  const T* kc = (const T*)a.k_cache + ((int64_t)g * MAPS + map) * d;
   const int64_t krow = (int64_t)a.kv_heads * MAPS * d, vrow_ = (int64_t)a.kv_heads * dv;
-  frag qf[MAPS][KS];
+  frag qf[KS];
   const frag zero = {};
-#pragma unroll
-  for (int m = 0; m < MAPS; ++m)
+  {
+    const T* qp = (const T*)a.q + t * a.q_token_stride + ((int64_t)(h0 + min(li, nh - 1)) * MAPS + map) * d;
 #pragma unroll
     for (int s = 0; s < KS; ++s) {
       const int i = 32 * s + 8 * lg;
-      const T* qp = (const T*)a.q + t * a.q_token_stride + ((int64_t)(h0 + min(li, nh - 1)) * MAPS + m) * d;
       const frag v = *reinterpret_cast<const frag*>(qp + min(i, d - 8));
-      qf[m][s] = i < d ? v : zero;
+      qf[s] = i < d ? v : zero;
     }
-  f32x4 acc[MAPS][VC];
-  float run_m[MAPS], run_l[MAPS];
-#pragma unroll
-  for (int m = 0; m < MAPS; ++m) {
-    run_m[m] = -INFINITY;
-    run_l[m] = 0.f;
-#pragma unroll
-    for (int c = 0; c < VC; ++c) acc[m][c] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
+  f32x4 acc[VC];
+  float run_m = -INFINITY, run_l = 0.f;
+#pragma unroll
+  for (int c = 0; c < VC; ++c) acc[c] = f32x4{0.f, 0.f, 0.f, 0.f};
   char* vsw = smd + wave * 32 * VP;
-  const int vch = dv / 8;
-  int vr_[VN], vo_[VN];
-  bool vl_[VN];
-#pragma unroll
-  for (int u = 0; u < VN; ++u) {
-    const int e = lane + 64 * u, ec = min(e, 32 * vch - 1);
-    vr_[u] = ec / vch;
-    vo_[u] = (ec - vr_[u] * vch) * 8;
-    vl_[u] = e < 32 * vch;
-  }
+  // a lane owns one chunk column of the V rows lane / VL + u * 64 / VL; columns past dv are left alone
+  const int vr0 = lane / VL, vc0 = (lane % VL) * 8;
+  const bool vlive = vc0 < dv;
+  const T* vc = (const T*)a.v_cache + (int64_t)g * dv + (vlive ? vc0 : 0);
+  char* vst = vsw + vr0 * VP + 2 * vc0;
   const bool cap = a.cap > 0.f;
   const float qmul = cap ? CA_LOG2E : a.scale * CA_LOG2E;
   const float k2 = cap ? 2.0f * CA_LOG2E * a.scale / a.cap : 0.f;
-  frag kf[2][MAPS][KS];
+  frag kf[2][KS];
   Vec<T, 8> vreg[VN];
   int slot = 0;                               // lane l & 31: the cache slot of key l & 31 of the tile whose rows come next
   auto load_slots = [&](int tile) { slot = table[min(tile * 32 + (lane & 31), len - 1)]; };
@@ -637,76 +630,70 @@ __global__ __launch_bounds__(256) void causal_attention_token_kernel(CaArgs a) {
     for (int hf = 0; hf < 2; ++hf) {
       const T* kp = kc + (int64_t)__shfl(slot, 16 * hf + li, 64) * krow;
 #pragma unroll
-      for (int m = 0; m < MAPS; ++m)
-#pragma unroll
-        for (int s = 0; s < KS; ++s) {
-          const int i = 32 * s + 8 * lg;
-          const frag v = *reinterpret_cast<const frag*>(kp + m * d + min(i, d - 8));
-          kf[hf][m][s] = i < d ? v : zero;
-        }
+      for (int s = 0; s < KS; ++s) {
+        const int i = 32 * s + 8 * lg;
+        const frag v = *reinterpret_cast<const frag*>(kp + min(i, d - 8));
+        kf[hf][s] = i < d ? v : zero;
+      }
     }
 #pragma unroll
-    for (int u = 0; u < VN; ++u) vreg[u] = ldvec<T, 8>(vc + (int64_t)__shfl(slot, vr_[u], 64) * vrow_ + vo_[u]);
+    for (int u = 0; u < VN; ++u) vreg[u] = ldvec<T, 8>(vc + (int64_t)__shfl(slot, vr0 + u * (64 / VL), 64) * vrow_);
   };
   const char* v_rd = vsw + VP * (4 * lg + (li >> 2)) + 8 * (li & 3);
-  int tile = tile_lo + wave;
+  int tile = tile_lo + stream;
   if (tile < tile_hi) {                       // wave-uniform
     load_slots(tile);
     load_rows();
-    load_slots(min(tile + 4, ntiles - 1));
+    load_slots(min(tile + STREAMS, ntiles - 1));
   }
-  for (; tile < tile_hi; tile += 4) {
+  for (; tile < tile_hi; tile += STREAMS) {
     // V to LDS (this wave's piece; a wave's LDS accesses stay in order), scores from the K fragments
+    if (vlive) {
 #pragma unroll
-    for (int u = 0; u < VN; ++u)
-      if (vl_[u]) lds_store16(vsw + vr_[u] * VP + 2 * vo_[u], vreg[u]);
-    f32x4 st[MAPS][2];
+      for (int u = 0; u < VN; ++u) lds_store16(vst + u * (64 / VL) * VP, vreg[u]);
+    }
+    f32x4 st[2];
 #pragma unroll
-    for (int m = 0; m < MAPS; ++m)
+    for (int hf = 0; hf < 2; ++hf) {
+      st[hf] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int hf = 0; hf < 2; ++hf) {
-        st[m][hf] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-        for (int s = 0; s < KS; ++s) st[m][hf] = Mfma<T>::run(kf[hf][m][s], qf[m][s], st[m][hf]);
-      }
-    if (tile + 4 < tile_hi) {                 // the next tile's rows are in flight during the rest
+      for (int s = 0; s < KS; ++s) st[hf] = Mfma<T>::run(kf[hf][s], qf[s], st[hf]);
+    }
+    if (tile + STREAMS < tile_hi) {           // the next tile's rows are in flight during the rest
       load_rows();
-      load_slots(min(tile + 8, ntiles - 1));
+      load_slots(min(tile + 2 * STREAMS, ntiles - 1));
     }
     const int lim = len - 1 - tile * 32 - 4 * lg;      // last visible key, relative to this lane's first
-    frag pb[MAPS];
+    float mloc = -INFINITY;
 #pragma unroll
-    for (int m = 0; m < MAPS; ++m) {
-      float mloc = -INFINITY;
+    for (int hf = 0; hf < 2; ++hf)
 #pragma unroll
-      for (int hf = 0; hf < 2; ++hf)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          float x = st[m][hf][r];
-          if (cap) x = ca_cap_fast(x, a.cap, k2);
-          x = 16 * hf + r > lim ? -INFINITY : x;
-          st[m][hf][r] = x;
-          mloc = fmaxf(mloc, x);
-        }
-      mloc = fmaxf(mloc, __shfl_xor(mloc, 16, 64));
-      mloc = fmaxf(mloc, __shfl_xor(mloc, 32, 64));
-      const float mnew = fmaxf(run_m[m], mloc * qmul);   // finite: a tile's first key is always visible
-      const float alpha = __builtin_amdgcn_exp2f(run_m[m] - mnew);
-      run_m[m] = mnew;
-      float psum = 0.f;
-#pragma unroll
-      for (int hf = 0; hf < 2; ++hf)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const float pe = __builtin_amdgcn_exp2f(__builtin_fmaf(st[m][hf][r], qmul, -mnew));
-          psum += pe;
-          pb[m][4 * hf + r] = (T)pe;
-        }
-      run_l[m] = run_l[m] * alpha + psum;     // this lane's keys alone; the lanes of a head are added at the end
-      if (__builtin_amdgcn_ballot_w64(alpha != 1.f) != 0) {
-#pragma unroll
-        for (int c = 0; c < VC; ++c) acc[m][c] *= alpha;
+      for (int r = 0; r < 4; ++r) {
+        float x = st[hf][r];
+        if (cap) x = ca_cap_fast(x, a.cap, k2);
+        x = 16 * hf + r > lim ? -INFINITY : x;
+        st[hf][r] = x;
+        mloc = fmaxf(mloc, x);
       }
+    mloc = fmaxf(mloc, __shfl_xor(mloc, 16, 64));
+    mloc = fmaxf(mloc, __shfl_xor(mloc, 32, 64));
+    const float mnew = fmaxf(run_m, mloc * qmul);      // finite: a tile's first key is always visible
+    const float alpha = __builtin_amdgcn_exp2f(run_m - mnew);
+    run_m = mnew;
+    float psum = 0.f;
+    frag pb;
+#pragma unroll
+    for (int hf = 0; hf < 2; ++hf)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float pe = __builtin_amdgcn_exp2f(__builtin_fmaf(st[hf][r], qmul, -mnew));
+        psum += pe;
+        pb[4 * hf + r] = (T)pe;
+      }
+    run_l = run_l * alpha + psum;             // this lane's keys alone; the lanes of a head are added at the end
+    if (__builtin_amdgcn_ballot_w64(alpha != 1.f) != 0) {
+#pragma unroll
+      for (int c = 0; c < VC; ++c) acc[c] *= alpha;
     }
     __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
     __builtin_amdgcn_wave_barrier();
@@ -715,89 +702,75 @@ __global__ __launch_bounds__(256) void causal_attention_token_kernel(CaArgs a) {
       typename TrRead<T>::v4 both[2];
       both[0] = TrRead<T>::run(reinterpret_cast<const T*>(v_rd + 32 * c));
       both[1] = TrRead<T>::run(reinterpret_cast<const T*>(v_rd + 16 * VP + 32 * c));
-#pragma unroll
-      for (int m = 0; m < MAPS; ++m) acc[m][c] = Mfma<T>::run(__builtin_bit_cast(frag, both), pb[m], acc[m][c]);
+      acc[c] = Mfma<T>::run(__builtin_bit_cast(frag, both), pb, acc[c]);
     }
     __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
     __builtin_amdgcn_wave_barrier();
   }
-  // ---- the four waves' results: common maximum, sums, then two rounds of adding through LDS
-#pragma unroll
-  for (int m = 0; m < MAPS; ++m) {
-    run_l[m] += __shfl_xor(run_l[m], 16, 64);
-    run_l[m] += __shfl_xor(run_l[m], 32, 64);
-    if (lg == 0) { red_m[wave][m][li] = run_m[m]; red_l[wave][m][li] = run_l[m]; }
-  }
+  // ---- the streams of a map: common maximum, sums, then rounds of adding through LDS; waves 0 (and 1: the second map) keep the result
+  run_l += __shfl_xor(run_l, 16, 64);
+  run_l += __shfl_xor(run_l, 32, 64);
+  if (lg == 0) { red_m[wave][li] = run_m; red_l[wave][li] = run_l; }
   __syncthreads();
-  float M[MAPS], L[MAPS];
+  float M = -INFINITY, L = 0.f;
 #pragma unroll
-  for (int m = 0; m < MAPS; ++m) {
-    M[m] = fmaxf(fmaxf(red_m[0][m][li], red_m[1][m][li]), fmaxf(red_m[2][m][li], red_m[3][m][li]));
-    const float Ms = M[m] == -INFINITY ? 0.f : M[m];
-    L[m] = 0.f;
+  for (int w = 0; w < STREAMS; ++w) M = fmaxf(M, red_m[w * MAPS + map][li]);
+  const float Ms = M == -INFINITY ? 0.f : M;
 #pragma unroll
-    for (int w = 0; w < 4; ++w) L[m] += red_l[w][m][li] * __builtin_amdgcn_exp2f(red_m[w][m][li] - Ms);
-    const float f = __builtin_amdgcn_exp2f(run_m[m] - Ms);
+  for (int w = 0; w < STREAMS; ++w) L += red_l[w * MAPS + map][li] * __builtin_amdgcn_exp2f(red_m[w * MAPS + map][li] - Ms);
+  const float f = __builtin_amdgcn_exp2f(run_m - Ms);
 #pragma unroll
-    for (int c = 0; c < VC; ++c) acc[m][c] *= f;
-  }
+  for (int c = 0; c < VC; ++c) acc[c] *= f;
   constexpr int XP = 16 * VC + 4;
   float* ex = reinterpret_cast<float*>(smd);
+  auto hand = [&](int piece, float factor) {
 #pragma unroll
-  for (int step = 2; step >= 1; step >>= 1) {
-    if (wave >= step && wave < 2 * step) {
+    for (int c = 0; c < VC; ++c) lds_store16(ex + (piece * 16 + li) * XP + 16 * c + 4 * lg, __builtin_bit_cast(Vec<float, 4>, acc[c] * factor));
+  };
+  auto take = [&](int piece, float sign) {
 #pragma unroll
-      for (int m = 0; m < MAPS; ++m)
+    for (int c = 0; c < VC; ++c) acc[c] += lds_load16<f32x4>(ex + (piece * 16 + li) * XP + 16 * c + 4 * lg) * sign;
+  };
 #pragma unroll
-        for (int c = 0; c < VC; ++c)
-          lds_store16(ex + (((wave - step) * MAPS + m) * 16 + li) * XP + 16 * c + 4 * lg, __builtin_bit_cast(Vec<float, 4>, acc[m][c]));
-    }
+  for (int step = 2; step >= MAPS; step >>= 1) {      // waves step .. 2 step - 1 onto waves 0 .. step - 1
+    if (wave >= step && wave < 2 * step) hand(wave - step, 1.f);
     __syncthreads();
-    if (wave < step) {
-#pragma unroll
-      for (int m = 0; m < MAPS; ++m)
-#pragma unroll
-        for (int c = 0; c < VC; ++c)
-          acc[m][c] += lds_load16<f32x4>(ex + ((wave * MAPS + m) * 16 + li) * XP + 16 * c + 4 * lg);
-    }
+    if (wave < step) take(wave, 1.f);
     __syncthreads();
   }
-  if (wave != 0) return;
   const int h = h0 + li;
   // lane: head li, columns 16 c + 4 lg + r
   if (a.num_splits > 1) {
-    if (li >= nh) return;
+    if (wave >= MAPS || li >= nh) return;
+    float* part = a.partial + ((((int64_t)split * a.tokens + t) * a.heads + h) * MAPS + map) * (dv + 2);
 #pragma unroll
-    for (int m = 0; m < MAPS; ++m) {
-      float* part = a.partial + ((((int64_t)split * a.tokens + t) * a.heads + h) * MAPS + m) * (dv + 2);
+    for (int c = 0; c < VC; ++c)
 #pragma unroll
-      for (int c = 0; c < VC; ++c)
-#pragma unroll
-        for (int r = 0; r < 4; ++r)
-          if (16 * c + 4 * lg < dv) part[16 * c + 4 * lg + r] = acc[m][c][r];
-      // the merge works with natural exponents
-      if (lg == 0) { part[dv] = M[m] == -INFINITY ? CA_NEG : M[m] * 0.6931471805599453f; part[dv + 1] = L[m]; }
-    }
+      for (int r = 0; r < 4; ++r)
+        if (16 * c + 4 * lg < dv) part[16 * c + 4 * lg + r] = acc[c][r];
+    // the merge works with natural exponents
+    if (lg == 0) { part[dv] = M == -INFINITY ? CA_NEG : M * 0.6931471805599453f; part[dv + 1] = L; }
     return;
   }
-  const float inv1 = L[0] > 0.f ? 1.0f / L[0] : 0.f;
-  float mul = inv1;
+  const float inv = L > 0.f ? 1.0f / L : 0.f;
+  float mul = inv;
   if constexpr (MAPS == 2) {
-    const float inv2 = L[1] > 0.f ? a.lambda / L[1] : 0.f;
+    if (wave == 1) hand(0, inv * a.lambda);
+    __syncthreads();
+    if (wave != 0) return;
+#pragma unroll
+    for (int c = 0; c < VC; ++c) acc[c] *= inv;
+    take(0, -1.f);
     float q2 = 0.f;
 #pragma unroll
     for (int c = 0; c < VC; ++c)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const float o = 16 * c + 4 * lg < dv ? acc[0][c][r] * inv1 - acc[1][c][r] * inv2 : 0.f;
-        acc[0][c][r] = o;
-        q2 += o * o;
-      }
+      for (int r = 0; r < 4; ++r) q2 += 16 * c + 4 * lg < dv ? acc[c][r] * acc[c][r] : 0.f;
     q2 += __shfl_xor(q2, 16, 64);
     q2 += __shfl_xor(q2, 32, 64);
     mul = a.out_scale / sqrtf(q2 / (float)dv + a.eps);
   }
-  if (li >= nh) return;
+  if (wave != 0 || li >= nh) return;
   const T* gt = (const T*)a.gate + t * a.gate_token_stride;
   if (a.gate != nullptr && !a.gate_per_feature) mul *= ca_sigmoid_fast(to_f32(gt[h]));
   T* op = (T*)a.out + t * a.out_token_stride + (int64_t)h * dv;
@@ -809,10 +782,10 @@ __global__ __launch_bounds__(256) void causal_attention_token_kernel(CaArgs a) {
     if (a.gate != nullptr && a.gate_per_feature) {
       const Vec<T, 4> z = ldvec<T, 4>(gt + (int64_t)h * dv + col);
 #pragma unroll
-      for (int r = 0; r < 4; ++r) w.v[r] = from_f32<T>(acc[0][c][r] * mul * ca_sigmoid_fast(to_f32(z.v[r])));
+      for (int r = 0; r < 4; ++r) w.v[r] = from_f32<T>(acc[c][r] * mul * ca_sigmoid_fast(to_f32(z.v[r])));
     } else {
 #pragma unroll
-      for (int r = 0; r < 4; ++r) w.v[r] = from_f32<T>(acc[0][c][r] * mul);
+      for (int r = 0; r < 4; ++r) w.v[r] = from_f32<T>(acc[c][r] * mul);
     }
     stvec<T, 4>(op + col, w);
   }
@@ -840,7 +813,7 @@ template <typename T, int KS, int VT, int MAPS> int launch_ca_tile(const CaArgs&
   return a.cap > 0.f ? go(causal_attention_tile_kernel<T, KS, VT, MAPS, true>) : go(causal_attention_tile_kernel<T, KS, VT, MAPS, false>);
 }
 template <typename T, int KS, int VC, int MAPS> int launch_ca_token(const CaArgs& a, hipStream_t st) {
-  constexpr size_t lds = ct_lds<VC, MAPS>();
+  constexpr size_t lds = ct_lds<VC>();
   const int rep = a.heads / a.kv_heads;
   const int64_t wgs = a.num_runs * a.kv_heads * ((rep + 15) / 16);
   MI355_REQUIRE(wgs < ((int64_t)1 << 31), MI355_ERR_UNSUPPORTED, "causal_attention: too many tokens");

@@ -1924,11 +1924,12 @@ def causal_attention_run_tokens(heads: int, kv_heads: int, maps: int, head_dim: 
 
 
 def causal_attention_splits(tokens: int, heads: int, kv_heads: int, max_len: Optional[int]) -> int:
-    """Key ranges per single token: about two workgroups per CU, at least 256 keys each (max_len None, a captured step: the launch
-    itself leaves ranges of shorter sequences empty)."""
+    """Key ranges per single token: one workgroup per CU, at least 512 keys each (max_len None, a captured step: the launch itself
+    leaves ranges of shorter sequences empty).  Measured on MI355X with heads of 128: from 128 workgroups on one range is as good as
+    two at 1024 keys and every further range costs more than it hides; 16 sequences of 8192 keys want four ranges, 4 want eight."""
     wgs = max(1, tokens * kv_heads * ((heads // kv_heads + 15) // 16))
-    n = max(1, min(32, 512 // wgs))
-    return n if max_len is None else max(1, min(n, (max_len + 255) // 256))
+    n = max(1, min(32, 256 // wgs))
+    return n if max_len is None else max(1, min(n, (max_len + 511) // 512))
 
 
 def causal_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, out: torch.Tensor, req_to_token: torch.Tensor,
