@@ -183,6 +183,8 @@ class Mi355AttnBackend(AttentionBackend):
 
     # ---- HIP-graph capture / replay (static shapes; nothing to refresh per replay) ----
     def init_cuda_graph_state(self, max_bs: int, max_num_tokens: int):
+        if self.is_layered:
+            return          # these kernels plan their own key ranges and bring their own scratch
         self._scratch(max_bs, MAX_KV_SPLITS)
         if self.sliding_window_size:
             self.graph_window_indptr = torch.zeros(max_bs + 1, dtype=torch.int32, device=self.device)
@@ -192,6 +194,10 @@ class Mi355AttnBackend(AttentionBackend):
     def init_forward_metadata_capture_cuda_graph(self, bs, num_tokens, req_pool_indices, seq_lens,
                                                  encoder_lens, forward_mode, spec_info):
         assert forward_mode.is_decode_or_idle(), "only decode is captured"
+        if self.is_layered:
+            self.forward_metadata = ForwardMetadata()
+            self.forward_metadata.latent_blocks = {}
+            return
         # one graph serves every step: split for the longest context the model can reach
         splits = self._plan_splits(bs, self.max_context_len)
         self.graph_num_splits[bs] = splits
@@ -208,6 +214,8 @@ class Mi355AttnBackend(AttentionBackend):
 
     def init_forward_metadata_replay_cuda_graph(self, bs, req_pool_indices, seq_lens, seq_lens_sum,
                                                 encoder_lens, forward_mode, spec_info, seq_lens_cpu):
+        if self.is_layered:
+            return
         # the captured kernels read req_to_token / seq_lens from the static buffers directly; only the
         # window gather of sliding-window models is refreshed (into the buffers the graph captured)
         if self.sliding_window_size:

@@ -222,6 +222,29 @@ def test_greedy_generation_through_the_scheduler(model, chunk, mixed):
         assert sch.num_prefill_batches > 3
 
 
+def test_capture_needs_nothing_of_the_other_families(model, monkeypatch):
+    """A library built for this family alone lacks the split-KV decode kernels: preparing, capturing and replaying a step must not ask
+    for their plan or counters."""
+    import cpu_ops
+    from sglang_custom_amd import build
+    from sglang_custom_amd.model_executor.forward_batch_info import ForwardMode
+
+    cfg, w = model
+    assert "attn_causal.hip" in build.FAMILY_SOURCES["Lomazen"] and "attn_decode.hip" not in build.FAMILY_SOURCES["Lomazen"]
+    mr = lu.build_runner(cfg, w)
+
+    def absent(*_a, **_k):
+        raise RuntimeError("not in this library")
+
+    monkeypatch.setattr(cpu_ops, "decode_num_splits", absent, raising=False)
+    b, two = mr.attn_backend, torch.ones(2, dtype=torch.int64)
+    b.init_cuda_graph_state(2, 2)
+    b.init_forward_metadata_capture_cuda_graph(2, 2, two, two, None, ForwardMode.DECODE, None)
+    assert b.forward_metadata is not None
+    b.init_forward_metadata_replay_cuda_graph(2, two, two, 2, None, ForwardMode.DECODE, None, two)
+    assert b._lse is None and b._tickets is None
+
+
 def test_planted_mistakes_show(model):
     """Each branch of the design left out of the oracle moves the logits far past the tolerance: what the comparisons above rest on."""
     cfg, w = model
