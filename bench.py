@@ -151,6 +151,7 @@ def measure_dominant_kernel(mr, bs, cfg, tp, dtype_bytes, quant=None):
     the same call the model makes -- bracketed by HIP events on the stream the kernels are launched on."""
     from sglang_custom_amd.layers.quantization.unquant import (QuantizedAct, decode_linear, decode_linear_deferred,
                                                               gate_up_silu_mul)
+    from sglang_custom_amd.model_executor.hip_graph_runner import collector_paused
     from sglang_custom_amd.ops_backend import get_ops
 
     dev = mr.device
@@ -192,7 +193,7 @@ def measure_dominant_kernel(mr, bs, cfg, tp, dtype_bytes, quant=None):
     one_pass()
     torch.cuda.synchronize()
     g = torch.cuda.CUDAGraph()   # replay from a graph: no host launch gaps inside the bracket
-    with torch.cuda.graph(g):
+    with collector_paused(), torch.cuda.graph(g):
         one_pass()
     reps = 5
     e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)

@@ -4,6 +4,8 @@ static input buffers -- the role of the reference's CudaGraphRunner
 :456, replay_prepare :626-700, replay :702-730).  ~330 kernel launches per step collapse into
 one graph launch; padded rows use seq_len fill value 1 and KV slot 0 (the sink row)."""
 import bisect
+import contextlib
+import gc
 from typing import Dict, List
 
 import torch
@@ -19,6 +21,21 @@ def get_batch_sizes_to_capture(max_bs: int) -> List[int]:
     if max_bs not in out:
         out.append(max_bs)
     return sorted(out)
+
+
+@contextlib.contextmanager
+def collector_paused():
+    """Python's cyclic collector runs now and not inside.  A model runner and its graph runner refer to each other, so graphs of a
+    runner that was dropped are freed by the collector, at whatever allocation sets it off; freeing a graph waits for the device,
+    which must not happen while a stream is being captured (the process is ended)."""
+    gc.collect()
+    was_on = gc.isenabled()
+    gc.disable()
+    try:
+        yield
+    finally:
+        if was_on:
+            gc.enable()
 
 
 class HipGraphRunner:
@@ -39,7 +56,8 @@ class HipGraphRunner:
         self.outputs: Dict[int, torch.Tensor] = {}
         self.pool = None
         model_runner.attn_backend.init_cuda_graph_state(self.max_bs, self.max_bs)
-        self.capture()
+        with collector_paused():
+            self.capture()
 
     def can_run(self, forward_batch: ForwardBatch) -> bool:
         return forward_batch.forward_mode.is_decode() and forward_batch.batch_size <= self.max_bs

@@ -115,8 +115,10 @@ def _rank_main(rank, world, port, queue, one_gpu_per_rank=False):
         torch.cuda.current_stream().wait_stream(side)
         torch.cuda.synchronize()
         dist.barrier()
+        from sglang_custom_amd.model_executor.hip_graph_runner import collector_paused
+
         graph = torch.cuda.CUDAGraph()
-        with ca.capture(), torch.cuda.graph(graph):
+        with collector_paused(), ca.capture(), torch.cuda.graph(graph):
             ca.all_reduce(a, out=oa)
             ca.all_reduce(b, out=ob)
         for rep in range(3):
@@ -462,8 +464,10 @@ def _ops_rank_main(rank, world, port, queue, one_gpu_per_rank=False):
                 g_out = torch.empty_like(x)
                 torch.cuda.synchronize()
                 dist.barrier()
+                from sglang_custom_amd.model_executor.hip_graph_runner import collector_paused
+
                 graph = torch.cuda.CUDAGraph()
-                with torch.cuda.graph(graph):                              # graph form
+                with collector_paused(), torch.cuda.graph(graph):          # graph form
                     ops.all_reduce_reg(fa, x, g_out)
                 h, o = ops.get_graph_buffer_ipc_meta(fa)
                 hs, os_ = gather((bytes(h), o))

@@ -12,6 +12,7 @@ import torch
 
 import cases
 from oracle import ops_ref
+from sglang_custom_amd.model_executor.hip_graph_runner import collector_paused
 
 pytestmark = pytest.mark.gpu
 DT = cases.DTYPES
@@ -1063,7 +1064,7 @@ def test_argmax_over_several_workgroups_per_row(ops):
     s.wait_stream(torch.cuda.current_stream())
     with torch.cuda.stream(s):
         gr = torch.cuda.CUDAGraph()
-        with torch.cuda.graph(gr, stream=s):
+        with collector_paused(), torch.cuda.graph(gr, stream=s):
             out = ops.argmax(x)
     torch.cuda.current_stream().wait_stream(s)
     for _ in range(3):

@@ -9,6 +9,7 @@ import torch
 
 import cases
 from oracle import ops_ref
+from sglang_custom_amd.model_executor.hip_graph_runner import collector_paused
 
 pytestmark = pytest.mark.gpu
 DEV = "cuda"
@@ -302,7 +303,7 @@ def test_per_sequence_split_plan_on_a_ragged_batch(ops, in_kernel_merge):
         ops.decode_attention_paged(q, kc, vc, out, r2t, pool, lt, al, ll, S, D ** -0.5, tickets=tickets, kv_chunk_keys=ck)
         torch.cuda.synchronize()
         gr = torch.cuda.CUDAGraph()
-        with torch.cuda.graph(gr, stream=s):
+        with collector_paused(), torch.cuda.graph(gr, stream=s):
             ops.decode_attention_paged(q, kc, vc, out, r2t, pool, lt, al, ll, S, D ** -0.5, tickets=tickets, kv_chunk_keys=ck)
     torch.cuda.current_stream().wait_stream(s)
     ck.fill_(1)          # too small for any sequence: every sequence falls back to the even 8-way cut

@@ -743,3 +743,40 @@ def test_input_token_logprobs_match_reference_vectors():
     golden = json.load(open(os.path.join(os.path.dirname(os.path.abspath(__file__)), "golden", "logprob.json")))
     cfg, w, dt, mr = _build(golden["preset"], "float32")
     cases.check_logprob_records(cases.run_logprob_scenarios(mr, golden), golden, 1e-4)
+
+
+def test_no_cyclic_garbage_is_freed_during_a_capture():
+    """Graphs of a dropped runner are cyclic garbage; freeing one while a stream is being captured ends the process.  What is garbage
+    before is freed before, what becomes garbage inside waits, and the collector's state comes back, also after an error."""
+    import gc
+    import weakref
+
+    from sglang_custom_amd.model_executor.hip_graph_runner import collector_paused
+
+    class Node:
+        pass
+
+    def cycle():
+        a, b = Node(), Node()
+        a.other, b.other = b, a
+        return weakref.ref(a)
+
+    assert gc.isenabled()
+    before = cycle()
+    with pytest.raises(RuntimeError):
+        with collector_paused():
+            assert before() is None
+            inside = cycle()
+            junk = [[] for _ in range(200000)]      # enough allocations to set a running collector off
+            assert len(junk) and inside() is not None and not gc.isenabled()
+            raise RuntimeError
+    assert gc.isenabled()
+    gc.collect()
+    assert inside() is None
+    gc.disable()
+    try:
+        with collector_paused():
+            pass
+        assert not gc.isenabled()
+    finally:
+        gc.enable()
