@@ -59,8 +59,8 @@ def test_mixture_of_squared_relu_experts(dtype, T, kw):
 @pytest.mark.parametrize("dtype", DTYPES)
 def test_rotation_norms_and_cache_rows(dtype):
     cases.check_frequencies()
-    for kw in (dict(), dict(rot=0), dict(interleaved=False), dict(interleaved=False, rot=6), dict(d=16, rot=16, W=24), dict(d=64, rot=64, R=8, S=2, W=160),
-               dict(d=48, rot=12, interleaved=False, unit_norm=False, R=8, S=4, W=192), dict(d=128, rot=64, interleaved=False, R=64, S=16, W=2048, T=3),
+    for kw in (dict(), dict(rot=0), dict(interleaved=False), dict(interleaved=False, rot=6), dict(d=16, rot=16, W=24), dict(d=64, rot=64, R=10, S=5, W=440),
+               dict(d=56, rot=20, interleaved=False, unit_norm=False, R=12, S=4, W=208), dict(d=128, rot=64, interleaved=False, R=64, S=16, W=2048, T=3),
                dict(d=256, rot=128, R=5, S=5, W=40), dict(d=7, rot=4, W=9, off=3), dict(d=24, rot=20, R=3, S=1, W=8), dict(d=33, rot=32, interleaved=False, W=5),
                dict(d=600, rot=2, R=2, S=1, W=8), dict(d=2, rot=2, R=1, S=1, W=1)):
         cases.check_rotate_write(ops(), DEV, dtype, **kw)
@@ -68,7 +68,7 @@ def test_rotation_norms_and_cache_rows(dtype):
 
 # head counts and widths: whole matrix-core tiles, widths padded to them, widths without 16-byte rows, one head, more heads than a
 # tile's columns or rows, widths past what the matrix-core kernels take
-SHAPES = [(8, 2, 1, 64, 80), (4, 2, 2, 48, 96), (16, 4, 1, 128, 128), (8, 2, 2, 128, 256), (6, 2, 1, 16, 24), (3, 3, 2, 40, 8), (1, 1, 1, 8, 8), (20, 1, 1, 72, 64),
+SHAPES = [(10, 5, 1, 64, 88), (6, 2, 2, 56, 104), (16, 4, 1, 128, 128), (8, 2, 2, 128, 256), (6, 2, 1, 16, 24), (3, 3, 2, 40, 8), (1, 1, 1, 8, 8), (20, 1, 1, 72, 64),
           (40, 2, 2, 24, 40), (140, 1, 1, 32, 16), (5, 5, 1, 11, 13), (4, 2, 2, 7, 20), (2, 1, 1, 256, 256), (2, 2, 1, 200, 136), (2, 1, 2, 136, 48), (3, 1, 1, 264, 300),
           (6, 3, 2, 64, 128), (12, 12, 1, 88, 120)]
 
@@ -85,7 +85,7 @@ def test_attention(dtype, H, G, maps, d, dv):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("kw", [dict(), dict(maps=2), dict(H=4, G=4, d=64, dv=32, page=32), dict(H=2, G=1, maps=2, d=48, dv=96, page=16)])
+@pytest.mark.parametrize("kw", [dict(), dict(maps=2), dict(H=4, G=4, d=64, dv=32, page=32), dict(H=2, G=1, maps=2, d=56, dv=104, page=16)])
 def test_attention_one_key_among_hundreds(dtype, kw):
     cases.check_attention_planted(ops(), DEV, dtype, **kw)
 
@@ -95,7 +95,7 @@ def test_score_cap_difference_batches_rotation(dtype):
     cases.check_score_cap(ops(), DEV, dtype)
     cases.check_score_cap(ops(), DEV, dtype, H=3, G=1, d=70, dv=9)
     cases.check_difference(ops(), DEV, dtype)
-    cases.check_difference(ops(), DEV, dtype, H=6, G=2, d=48, dv=96)
+    cases.check_difference(ops(), DEV, dtype, H=6, G=2, d=56, dv=104)
     for maps in (1, 2):
         cases.check_batch_of_unequal(ops(), DEV, dtype, maps=maps)
         cases.check_batch_of_unequal(ops(), DEV, dtype, maps=maps, H=8, G=8, d=64, dv=128)
